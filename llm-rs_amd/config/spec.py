@@ -63,6 +63,9 @@ class ModelSpec:
     # patterns (fnmatch) of tensor names this architecture's files may hold although the model reads none of them
     ignorable_tensors: Tuple[str, ...] = ()
     embedding_scale: float = 1.0    # the token table's rows are multiplied by this on their way into the stream
+    # > 0: a vector of the token's position p is added to them at the start, feature 2i the sine and 2i + 1 the cosine of
+    # p * base^(-2i / hidden_size) with this base
+    position_wave_base: float = 0.0
     logit_scale: float = 1.0        # logits are multiplied by this, and then,
     logit_softcap: float = 0.0      # if > 0, bent into (-cap, cap): cap * tanh(logit / cap)
     # The residual stream kept as this many copies, all equal to the embedding at the start and summed before the
@@ -75,6 +78,8 @@ class ModelSpec:
             raise ValueError("a model needs at least one layer")
         if not 1 <= self.streams <= 16:
             raise ValueError(f"the residual stream has 1 to 16 copies, not {self.streams}")
+        if self.position_wave_base < 0 or (self.position_wave_base > 0 and self.streams > 1):
+            raise ValueError("a position vector has a positive base, and goes with a stream in one copy")
         for i, layer in enumerate(self.layers):
             names = [e.name for e in layer.extra]
             for e in layer.extra:

@@ -26,14 +26,33 @@ struct AttnArgs {
     // its one rounding.
     const float* gate;
     int gate_stride, gate_per;
+    // > 0 (window 0): positions lie in chunks of so many, counted from the request's position 0, and a query sees the keys
+    // of its own chunk only: key j is visible to the query at i when j <= i and j >= i - i % mask_chunk.
+    int mask_chunk;
+    // 2: differential attention.  A head's row of q and a key's row hold two halves of head_dim / 2 features; each half is
+    // an attention (a map) of its own over the same values, and with a1, a2 the maps' results the head's output is
+    //   o = a1 - diff_lambda a2,   o / sqrt(mean(o^2) + diff_eps) * diff_scale        (32-bit, before gate and rounding)
+    // 1: head_dim features are one map.
+    int maps;
+    float diff_lambda, diff_eps, diff_scale;
 };
 // Whether a call is the plain one (values as wide as keys, no distance penalty, no soft cap, no kept first keys) that
 // every kernel file takes.
 static inline bool attn_is_plain(const AttnArgs& a) {
-    return a.v_dim == a.head_dim && a.dist_r1 == nullptr && a.softcap <= 0.0f && (a.keep_first <= 0 || a.window <= 0) && a.sink == nullptr && a.gate == nullptr;
+    return a.v_dim == a.head_dim && a.dist_r1 == nullptr && a.softcap <= 0.0f && (a.keep_first <= 0 || a.window <= 0) && a.sink == nullptr && a.gate == nullptr &&
+           a.mask_chunk <= 0 && a.maps == 1;
 }
-// The first key of the window of the query at `pos`, and how many of the first keys lie before it and stay visible.
+// How many keys a query sees at most (0: all that came before it).
+static inline int attn_reach(const AttnArgs& a) { return a.mask_chunk > 0 ? a.mask_chunk : a.window; }
+// Chunks of `chunk` keys that a single token's keys can lie in, of `max_chunks` over the whole length.
+static inline int attn_chunks_seen(const AttnArgs& a, int max_chunks, int chunk) {
+    int reach = attn_reach(a);
+    return reach > 0 && (reach - 1) / chunk + 2 < max_chunks ? (reach - 1) / chunk + 2 : max_chunks;
+}
+// The first key of the window (or the chunk) of the query at `pos`, and how many of the first keys lie before it and
+// stay visible.  It never falls as `pos` rises.
 __host__ __device__ static inline int attn_window_lo(const AttnArgs& a, int pos) {
+    if (a.mask_chunk > 0) return pos > 0 ? pos - pos % a.mask_chunk : 0;
     return (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
 }
 __host__ __device__ static inline int attn_kept_before(const AttnArgs& a, int lo) {

@@ -20,6 +20,8 @@
 // 16-byte aligned rows; otherwise the caller keeps to the walk.
 // Entries with one token are shared out over waves by key range on the same products (attn_f32_split_kernel): a
 // decode step in 32-bit reads its keys and values once for all heads of a kv head, 16 bytes a lane.
+// Differential attention (MAPS 2): neighbouring columns are the two maps of a head, c even the first; a column's query is
+// zero in the other map's features, and the columns' results are made one at the end (or by the merge).
 // Formulas: shaders/ops.metal:636-758 (scale after the dot, causal bound, softmax, weighted sum).
 #include "attention.h"
 #include "cache_layout.h"
@@ -120,7 +122,18 @@ __device__ __forceinline__ void f32_walk(const f32x4 (&qf)[HD / 8], const float*
     }
 }
 
-template <int HD>
+// Values 8j + 4h .. 8j + 4h + 3 of the query at `qp` (which points 4h into its row), those of the map's own features.
+template <int HD, int MAPS>
+__device__ __forceinline__ void f32_query(f32x4 (&qf)[HD / 8], const float* qp, int map) {
+#pragma unroll
+    for (int j = 0; j < HD / 8; ++j) {
+        qf[j] = *(const f32x4*)(qp + 8 * j);
+        if constexpr (MAPS == 2)
+            if ((8 * j >= HD / 2 ? 1 : 0) != map) qf[j] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    }
+}
+
+template <int HD, int MAPS>
 __global__ __launch_bounds__(256) void attn_f32_tiles_kernel(const float* __restrict__ q, float* __restrict__ out,
                                                              const float* __restrict__ kc, const float* __restrict__ vc,
                                                              const int* __restrict__ block_table,
@@ -139,19 +152,17 @@ __global__ __launch_bounds__(256) void attn_f32_tiles_kernel(const float* __rest
     int tq = c / G, hg = c - tq * G;
     bool cvalid = tq < ntok;
     int token = tok0 + min(tq, ntok - 1);
-    int head = kvh * G + hg;
+    int head = (kvh * G + hg) / MAPS;              // (G: columns of a kv head)
     int pos = cvalid ? positions[token] : -1;
-    int lo = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+    int lo = attn_window_lo(a, pos);
     int last = positions[tok0 + ntok - 1], first = positions[tok0];
     int t_end = last + 1;
-    int t_begin = ((a.window > 0 && first + 1 > a.window) ? first + 1 - a.window : 0) & ~31;
+    int t_begin = attn_window_lo(a, first) & ~31;
     const int* table = block_table + (size_t)e * a.table_width;
 
     // this lane's part of its column's query: values 8j + 4h .. 8j + 4h + 3
     f32x4 qf[HD / 8];
-    const float* qp = q + (size_t)token * a.q_stride + (size_t)head * HD + 4 * h;
-#pragma unroll
-    for (int j = 0; j < HD / 8; ++j) qf[j] = *(const f32x4*)(qp + 8 * j);
+    f32_query<HD, MAPS>(qf, q + (size_t)token * a.q_stride + (size_t)head * HD + 4 * h, c % MAPS);
     f32x16 O[HD / 32];
 #pragma unroll
     for (int dt = 0; dt < HD / 32; ++dt)
@@ -162,8 +173,22 @@ __global__ __launch_bounds__(256) void attn_f32_tiles_kernel(const float* __rest
     // pass the mask there)
     if (a.keep_first > 0 && t_begin > 0) f32_walk<HD>(qf, kc, vc, table, a, kvh, c, h, pos, lo, 0, min(a.keep_first, t_begin), O, m, l);
     f32_walk<HD>(qf, kc, vc, table, a, kvh, c, h, pos, lo, t_begin, t_end, O, m, l);
-    if (!cvalid) return;
     float inv = 1.0f / (l + attn_sink_term_base2(a, head, m));      // (the sum is complete here: the sink joins it once)
+    if constexpr (MAPS == 2) {
+        float ss = 0.0f;
+#pragma unroll
+        for (int dt = 0; dt < HD / 32; ++dt)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                float mine = O[dt][i] * inv, other = __shfl_xor(mine, 1, 64);      // the column beside this one is the head's other map
+                float o = (c & 1) ? other - a.diff_lambda * mine : mine - a.diff_lambda * other;
+                O[dt][i] = o;
+                ss = fmaf(o, o, ss);
+            }
+        ss += swap_halves(ss);
+        inv = 1.0f / sqrtf(ss / (float)HD + a.diff_eps) * a.diff_scale;
+    }
+    if (!cvalid || c % MAPS) return;
     float* op = out + (size_t)token * a.out_stride + (size_t)head * HD + 4 * h;
 #pragma unroll
     for (int dt = 0; dt < HD / 32; ++dt)
@@ -181,7 +206,7 @@ __global__ __launch_bounds__(256) void attn_f32_tiles_kernel(const float* __rest
 // once for all of them, 16 bytes a lane, which is what this step is bound by).  It leaves what the walk of
 // attention_generic.hip leaves for such a chunk, where that file's merge finds it: the maximum (natural logarithm's
 // scale), the sum and the weighted values of each head, [entry][head][chunk][2 + head_dim].
-template <int HD>
+template <int HD, int MAPS>
 __global__ __launch_bounds__(64) void attn_f32_split_kernel(const float* __restrict__ q, float* __restrict__ partial,
                                                             const float* __restrict__ kc, const float* __restrict__ vc,
                                                             const int* __restrict__ block_table,
@@ -192,18 +217,16 @@ __global__ __launch_bounds__(64) void attn_f32_split_kernel(const float* __restr
     int token = q_starts[e];
     if (q_starts[e + 1] - token != 1) return;
     int pos_t = seq_lens[e] - 1;                  // an entry with one token: its position is its length less one
-    int lo = (a.window > 0 && pos_t + 1 > a.window) ? pos_t + 1 - a.window : 0;
+    int lo = attn_window_lo(a, pos_t);
     int first = lo / F32_SPLIT_CHUNK;
     if (ch > pos_t / F32_SPLIT_CHUNK - first) return;
     int begin = max(lo, (first + ch) * F32_SPLIT_CHUNK), end = min(pos_t + 1, (first + ch + 1) * F32_SPLIT_CHUNK);
     bool cvalid = c < G;
-    int head = kvh * G + min(c, G - 1);
+    int column = kvh * G + min(c, G - 1), head = column / MAPS;         // (G: columns of a kv head; see the partial results' layout)
     int pos = cvalid ? pos_t : -1;
     const int* table = block_table + (size_t)e * a.table_width;
     f32x4 qf[HD / 8];
-    const float* qp = q + (size_t)token * a.q_stride + (size_t)head * HD + 4 * h;
-#pragma unroll
-    for (int j = 0; j < HD / 8; ++j) qf[j] = *(const f32x4*)(qp + 8 * j);
+    f32_query<HD, MAPS>(qf, q + (size_t)token * a.q_stride + (size_t)head * HD + 4 * h, c % MAPS);
     f32x16 O[HD / 32];
 #pragma unroll
     for (int dt = 0; dt < HD / 32; ++dt)
@@ -214,7 +237,7 @@ __global__ __launch_bounds__(64) void attn_f32_split_kernel(const float* __restr
         f32_walk<HD>(qf, kc, vc, table, a, kvh, c, h, pos, lo, 0, min(a.keep_first, begin & ~31), O, m, l);
     f32_walk<HD>(qf, kc, vc, table, a, kvh, c, h, pos, lo, begin & ~31, end, O, m, l);
     if (!cvalid) return;
-    float* pp = partial + ((size_t)(e * a.n_heads + head) * max_chunks + ch) * (HD + 2);
+    float* pp = partial + ((size_t)(e * a.n_heads * MAPS + column) * max_chunks + ch) * (HD + 2);
     if (h == 0) { pp[0] = m * 0.69314718055994531f; pp[1] = l; }
     // this lane holds features dt * 32 + 8 g + 4 h + j of its column (rows of 2 + head_dim floats: 8-byte aligned)
 #pragma unroll
@@ -233,7 +256,7 @@ __global__ __launch_bounds__(64) void attn_f32_split_kernel(const float* __restr
 int llmrs_attention_f32_mfma(hipStream_t stream, const float* q, float* out, const float* k_cache, const float* v_cache,
                              const int* block_table, const int* positions, const int* q_starts, int n_entries,
                              int skip_single, const AttnArgs& a) {
-    int G = a.n_heads / a.n_kv_heads;
+    int G = a.n_heads / a.n_kv_heads * a.maps;
     if (a.v_dim != a.head_dim || a.dist_r1 != nullptr) return 0;
     if (a.head_dim % 32 || a.head_dim > 256 || a.page_size % 4 || G > 32 || q_starts == nullptr) return 0;
     if (a.q_stride % 4 || a.out_stride % 4 || ((uintptr_t)q & 15) || ((uintptr_t)out & 15) || ((uintptr_t)k_cache & 15) ||
@@ -244,9 +267,11 @@ int llmrs_attention_f32_mfma(hipStream_t stream, const float* q, float* out, con
     long blocks = ((tiles + 3) / 4) * a.n_kv_heads;
     if (blocks > 0x7fffffffL) return 0;
     switch (a.head_dim) {
-#define CASE(HD) case HD: attn_f32_tiles_kernel<HD><<<(int)blocks, 256, 0, stream>>>(q, out, k_cache, v_cache, block_table, positions, q_starts, n_entries, a, G, tpt, skip_single); break;
+#define TILES(HD, MM) attn_f32_tiles_kernel<HD, MM><<<(int)blocks, 256, 0, stream>>>(q, out, k_cache, v_cache, block_table, positions, q_starts, n_entries, a, G, tpt, skip_single)
+#define CASE(HD) case HD: if (a.maps == 2) TILES(HD, 2); else TILES(HD, 1); break;
         CASE(32) CASE(64) CASE(96) CASE(128) CASE(160) CASE(192) CASE(224) CASE(256)
 #undef CASE
+#undef TILES
         default: return 0;
     }
     hipError_t err = hipGetLastError();
@@ -262,7 +287,7 @@ int llmrs_attention_f32_mfma(hipStream_t stream, const float* q, float* out, con
 int llmrs_attention_f32_mfma_split(hipStream_t stream, const float* q, float* partial, const float* k_cache, const float* v_cache,
                                    const int* block_table, const int* q_starts, const int* seq_lens, int n_entries,
                                    int max_chunks, const AttnArgs& a) {
-    int G = a.n_heads / a.n_kv_heads;
+    int G = a.n_heads / a.n_kv_heads * a.maps;
     if (a.v_dim != a.head_dim || a.dist_r1 != nullptr) return 0;
     if (a.head_dim % 32 || a.head_dim > 256 || a.page_size % 4 || G > 32 || q_starts == nullptr || seq_lens == nullptr) return 0;
     if (a.q_stride % 4 || ((uintptr_t)q & 15) || ((uintptr_t)k_cache & 15) || ((uintptr_t)v_cache & 15) || ((uintptr_t)partial & 7))
@@ -270,9 +295,11 @@ int llmrs_attention_f32_mfma_split(hipStream_t stream, const float* q, float* pa
     if (n_entries > 65535 || a.n_kv_heads > 65535 || max_chunks > 65535 || max_chunks < 1) return 0;
     dim3 grid(n_entries, a.n_kv_heads, max_chunks);
     switch (a.head_dim) {
-#define CASE(HD) case HD: attn_f32_split_kernel<HD><<<grid, 64, 0, stream>>>(q, partial, k_cache, v_cache, block_table, q_starts, seq_lens, max_chunks, a, G); break;
+#define SPLIT(HD, MM) attn_f32_split_kernel<HD, MM><<<grid, 64, 0, stream>>>(q, partial, k_cache, v_cache, block_table, q_starts, seq_lens, max_chunks, a, G)
+#define CASE(HD) case HD: if (a.maps == 2) SPLIT(HD, 2); else SPLIT(HD, 1); break;
         CASE(32) CASE(64) CASE(96) CASE(128) CASE(160) CASE(192) CASE(224) CASE(256)
 #undef CASE
+#undef SPLIT
         default: return 0;
     }
     hipError_t err = hipGetLastError();

@@ -8,6 +8,8 @@
 // o = sum_j softmax_j v_j, divided by the sum at the end.  The mask is the loop's
 // bound.  This is the reference's paged_attention (shaders/ops.metal:636-758;
 // causal_len of :673-674 equals p + 1) with a tile of 64 keys, one per lane.
+// Or lo is the first position of the query's own chunk (a mask in chunks).  Differential attention (MAPS 2) walks the
+// same keys and values twice, once for each half of the head's features, and makes the two results one at the end.
 // Tiles start at lo, so for a given query the order of every sum is fixed: it
 // does not depend on the batch or on how the prompt was cut.  A decoding request's
 // keys are shared out over waves in chunks aligned to absolute positions and the
@@ -24,12 +26,13 @@
 
 // One wave walks the keys [begin, end) of its request for the query in `qs`, a tile of 64 keys at a
 // time (one key per lane), and folds them into the running maximum m, sum l and acc (lane's
-// features d = lane + 64 i, not yet divided by l).  VEC: head_dim % 4 == 0, a key's row is read four
-// elements at a load; the sums are the same either way.
+// features d = lane + 64 i, not yet divided by l).  The scores run over the features [d0, d0 + dn) of
+// the query and of a key's row (all of them, or those of a map).  VEC: d0 and dn are multiples of 4 and rows
+// are whole pieces of four, a key's row is read four elements at a load; the sums are the same either way.
 template <class T, bool VEC>
 __device__ __forceinline__ void walk_keys(const float* qs, const T* __restrict__ k_cache, const T* __restrict__ v_cache,
                                           const int* __restrict__ table, const AttnArgs& a, int kvh, int h, int pos,
-                                          int begin, int end, float& m, float& l, float (&acc)[MAX_HEAD_DIM / 64]) {
+                                          int begin, int end, int d0, int dn, float& m, float& l, float (&acc)[MAX_HEAD_DIM / 64]) {
     int lane = threadIdx.x, hd = a.head_dim, vd = a.v_dim, ps = a.page_size;
     // the distance penalty of this head (query at `pos`): r1 ln(1 + r2 (pos - j)), or none
     const bool far = a.dist_r1 != nullptr;
@@ -46,14 +49,14 @@ __device__ __forceinline__ void walk_keys(const float* qs, const T* __restrict__
             const T* kp = k_cache + k_cache_index(page, kvh, off, 0, a.n_kv_heads, ps, hd);
             float dot = 0.0f;
             if constexpr (VEC) {
-                for (int d = 0; d < hd; d += 4) {
+                for (int d = d0; d < d0 + dn; d += 4) {
                     float kv[4];
                     load4(kp + d, kv);
 #pragma unroll
                     for (int i = 0; i < 4; ++i) dot = fmaf(qs[d + i], kv[i], dot);
                 }
             } else {
-                for (int d = 0; d < hd; ++d) dot = fmaf(qs[d], to_f32(kp[d]), dot);
+                for (int d = d0; d < d0 + dn; ++d) dot = fmaf(qs[d], to_f32(kp[d]), dot);
             }
             s = dot * a.scale;
             if (a.softcap > 0.0f) s = a.softcap * tanhf(s / a.softcap);
@@ -80,8 +83,25 @@ __device__ __forceinline__ void walk_keys(const float* qs, const T* __restrict__
     }
 }
 
+// What a head's output is, from its maps' results (in acc, already divided): lane's features d = lane + 64 i, into acc[0].
+template <int MAPS>
+__device__ __forceinline__ void combine_maps(float (&acc)[MAPS][MAX_HEAD_DIM / 64], const AttnArgs& a) {
+    if constexpr (MAPS == 2) {
+        float ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
+            float o = ((int)threadIdx.x + 64 * i) < a.v_dim ? acc[0][i] - a.diff_lambda * acc[1][i] : 0.0f;
+            ss = fmaf(o, o, ss);
+            acc[0][i] = o;
+        }
+        float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.v_dim + a.diff_eps) * a.diff_scale;
+#pragma unroll
+        for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) acc[0][i] *= inv;
+    }
+}
+
 // skip_single: tokens of entries that bring one token are left to the split kernels below.
-template <class T, bool VEC>
+template <class T, bool VEC, int MAPS>
 __global__ __launch_bounds__(64) void attention_generic_kernel(
     const T* __restrict__ q, T* __restrict__ out, const T* __restrict__ k_cache, const T* __restrict__ v_cache,
     const int* __restrict__ block_table, const int* __restrict__ token_entry, const int* __restrict__ positions,
@@ -98,35 +118,43 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
     for (int d = lane; d < hd; d += 64) qs[d] = to_f32(qrow[d]);
     __syncthreads();
 
-    int lo = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
-    float m = -INFINITY, l = 0.0f;
-    float acc[MAX_HEAD_DIM / 64] = {};
+    int lo = attn_window_lo(a, pos);
     int kept = attn_kept_before(a, lo);         // first keys that the window has passed and that stay visible
-    if (kept > 0) walk_keys<T, VEC>(qs, k_cache, v_cache, table, a, kvh, h, pos, 0, kept, m, l, acc);
-    walk_keys<T, VEC>(qs, k_cache, v_cache, table, a, kvh, h, pos, lo, pos + 1, m, l, acc);
+    const int dn = hd / MAPS;
+    float acc[MAPS][MAX_HEAD_DIM / 64] = {};
+#pragma unroll
+    for (int map = 0; map < MAPS; ++map) {
+        float m = -INFINITY, l = 0.0f;
+        if (kept > 0) walk_keys<T, VEC>(qs, k_cache, v_cache, table, a, kvh, h, pos, 0, kept, map * dn, dn, m, l, acc[map]);
+        walk_keys<T, VEC>(qs, k_cache, v_cache, table, a, kvh, h, pos, lo, pos + 1, map * dn, dn, m, l, acc[map]);
+        l += attn_sink_term(a, h, m);
+#pragma unroll
+        for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) acc[map][i] /= l;
+    }
+    combine_maps<MAPS>(acc, a);
     T* orow = out + (size_t)t * a.out_stride + (size_t)h * a.v_dim;
-    l += attn_sink_term(a, h, m);
 #pragma unroll
     for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
         int d = lane + 64 * i;
-        if (d < a.v_dim) orow[d] = from_f32<T>(acc[i] / l * attn_gate(a, t, h, d));
+        if (d < a.v_dim) orow[d] = from_f32<T>(acc[0][i] * attn_gate(a, t, h, d));
     }
 }
 
 // Entries with one token (decoding): a wave for each (entry, head, chunk of GENERIC_CHUNK keys), so
 // that a long context is read by many waves at once.  Chunks are aligned to absolute positions.
-// partial: [(entry * n_heads + head) * max_chunks + chunk][head_dim + 2] = m, l, acc (not divided).
-template <class T, bool VEC>
+// partial: [(entry * columns + column) * max_chunks + chunk][v_dim + 2] = m, l, acc (not divided); a column is a head, or
+// with two maps a map of a head (column = 2 head + map).
+template <class T, bool VEC, int MAPS>
 __global__ __launch_bounds__(64) void attention_generic_split_kernel(
     const T* __restrict__ q, float* __restrict__ partial, const T* __restrict__ k_cache, const T* __restrict__ v_cache,
     const int* __restrict__ block_table, const int* __restrict__ q_starts, const int* __restrict__ seq_lens,
     int max_chunks, AttnArgs a) {
     __shared__ float qs[MAX_HEAD_DIM];
-    int e = blockIdx.x, h = blockIdx.y, ch = blockIdx.z, lane = threadIdx.x;
+    int e = blockIdx.x, column = blockIdx.y, h = column / MAPS, ch = blockIdx.z, lane = threadIdx.x;
     int t = q_starts[e];
     if (q_starts[e + 1] - t != 1) return;
     int pos = seq_lens[e] - 1;                    // an entry with one token: its position is its length less one
-    int lo = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+    int lo = attn_window_lo(a, pos);
     int first = lo / GENERIC_CHUNK;
     if (ch > pos / GENERIC_CHUNK - first) return;
     int begin = max(lo, (first + ch) * GENERIC_CHUNK), end = min(pos + 1, (first + ch + 1) * GENERIC_CHUNK);
@@ -137,10 +165,11 @@ __global__ __launch_bounds__(64) void attention_generic_split_kernel(
     __syncthreads();
     float m = -INFINITY, l = 0.0f;
     float acc[MAX_HEAD_DIM / 64] = {};
+    const int dn = hd / MAPS, d0 = (column % MAPS) * dn;
     int kept = ch == 0 ? attn_kept_before(a, lo) : 0;      // the first chunk's wave also takes the kept first keys
-    if (kept > 0) walk_keys<T, VEC>(qs, k_cache, v_cache, block_table + (size_t)e * a.table_width, a, kvh, h, pos, 0, kept, m, l, acc);
-    walk_keys<T, VEC>(qs, k_cache, v_cache, block_table + (size_t)e * a.table_width, a, kvh, h, pos, begin, end, m, l, acc);
-    float* pp = partial + ((size_t)(e * a.n_heads + h) * max_chunks + ch) * (a.v_dim + 2);
+    if (kept > 0) walk_keys<T, VEC>(qs, k_cache, v_cache, block_table + (size_t)e * a.table_width, a, kvh, h, pos, 0, kept, d0, dn, m, l, acc);
+    walk_keys<T, VEC>(qs, k_cache, v_cache, block_table + (size_t)e * a.table_width, a, kvh, h, pos, begin, end, d0, dn, m, l, acc);
+    float* pp = partial + ((size_t)(e * a.n_heads * MAPS + column) * max_chunks + ch) * (a.v_dim + 2);
     if (lane == 0) { pp[0] = m; pp[1] = l; }
 #pragma unroll
     for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
@@ -249,7 +278,7 @@ __global__ __launch_bounds__(64) void attention_generic_group_tokens_kernel(
     const T* qrow = q + (size_t)t * a.q_stride + (size_t)kvh * G * hd;      // the kv head's G heads lie side by side
     for (int d = lane; d < G * hd; d += 64) qs[d] = to_f32(qrow[d]);
     __syncthreads();
-    int lo = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+    int lo = attn_window_lo(a, pos);
     float m[G], l[G], acc[G][NACC];
 #pragma unroll
     for (int g = 0; g < G; ++g) {
@@ -284,7 +313,7 @@ __global__ __launch_bounds__(64) void attention_generic_group_kernel(
     int t = q_starts[e];
     if (q_starts[e + 1] - t != 1) return;
     int pos = seq_lens[e] - 1;                    // an entry with one token: its position is its length less one
-    int lo = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+    int lo = attn_window_lo(a, pos);
     int first = lo / GENERIC_CHUNK;
     if (ch > pos / GENERIC_CHUNK - first) return;
     int begin = max(lo, (first + ch) * GENERIC_CHUNK), end = min(pos + 1, (first + ch + 1) * GENERIC_CHUNK);
@@ -316,7 +345,7 @@ __global__ __launch_bounds__(64) void attention_generic_group_kernel(
 
 // One wave for each (entry, head) adds the chunks up.  The chunks' maxima and sums are read 64 at a time, a lane
 // each; the weighted values are added chunk by chunk in ascending order, four chunks' rows asked for at a time.
-template <class T>
+template <class T, int MAPS>
 __global__ __launch_bounds__(64) void attention_generic_merge_kernel(
     const float* __restrict__ partial, T* __restrict__ out, const int* __restrict__ q_starts,
     const int* __restrict__ seq_lens, int max_chunks, AttnArgs a) {
@@ -324,53 +353,59 @@ __global__ __launch_bounds__(64) void attention_generic_merge_kernel(
     int t = q_starts[e];
     if (q_starts[e + 1] - t != 1) return;
     int pos = seq_lens[e] - 1;
-    int lo = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+    int lo = attn_window_lo(a, pos);
     int n_chunks = pos / GENERIC_CHUNK - lo / GENERIC_CHUNK + 1;
-    const float* pp = partial + (size_t)(e * a.n_heads + h) * max_chunks * (hd + 2);
     const size_t stride = hd + 2;
-    float M = -INFINITY;
-    for (int ch = lane; ch < n_chunks; ch += 64) M = fmaxf(M, pp[(size_t)ch * stride]);
-    M = wave_max(M);
-    float L = 0.0f;
-    float o[MAX_HEAD_DIM / 64] = {};
-    for (int base = 0; base < n_chunks; base += 64) {
-        int mine = base + lane;
-        float w_mine = mine < n_chunks ? expf(pp[(size_t)mine * stride] - M) : 0.0f;
-        float l_mine = mine < n_chunks ? pp[(size_t)mine * stride + 1] * w_mine : 0.0f;
-        L += wave_sum(l_mine);
-        int n = min(64, n_chunks - base);
-        int j = 0;
-        for (; j + 4 <= n; j += 4) {
-            float v[4][MAX_HEAD_DIM / 64];
+    float o[MAPS][MAX_HEAD_DIM / 64] = {};
 #pragma unroll
-            for (int u = 0; u < 4; ++u)
+    for (int map = 0; map < MAPS; ++map) {
+        const float* pp = partial + (size_t)((e * a.n_heads + h) * MAPS + map) * max_chunks * stride;
+        float M = -INFINITY;
+        for (int ch = lane; ch < n_chunks; ch += 64) M = fmaxf(M, pp[(size_t)ch * stride]);
+        M = wave_max(M);
+        float L = 0.0f;
+        for (int base = 0; base < n_chunks; base += 64) {
+            int mine = base + lane;
+            float w_mine = mine < n_chunks ? expf(pp[(size_t)mine * stride] - M) : 0.0f;
+            float l_mine = mine < n_chunks ? pp[(size_t)mine * stride + 1] * w_mine : 0.0f;
+            L += wave_sum(l_mine);
+            int n = min(64, n_chunks - base);
+            int j = 0;
+            for (; j + 4 <= n; j += 4) {
+                float v[4][MAX_HEAD_DIM / 64];
+#pragma unroll
+                for (int u = 0; u < 4; ++u)
+#pragma unroll
+                    for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
+                        int d = lane + 64 * i;
+                        v[u][i] = d < hd ? pp[(size_t)(base + j + u) * stride + 2 + d] : 0.0f;
+                    }
+#pragma unroll
+                for (int u = 0; u < 4; ++u) {
+                    float w = __shfl(w_mine, j + u, 64);
+#pragma unroll
+                    for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) o[map][i] = fmaf(v[u][i], w, o[map][i]);
+                }
+            }
+            for (; j < n; ++j) {
+                float w = __shfl(w_mine, j, 64);
 #pragma unroll
                 for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
                     int d = lane + 64 * i;
-                    v[u][i] = d < hd ? pp[(size_t)(base + j + u) * stride + 2 + d] : 0.0f;
+                    if (d < hd) o[map][i] = fmaf(pp[(size_t)(base + j) * stride + 2 + d], w, o[map][i]);
                 }
-#pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                float w = __shfl(w_mine, j + u, 64);
-#pragma unroll
-                for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) o[i] = fmaf(v[u][i], w, o[i]);
             }
         }
-        for (; j < n; ++j) {
-            float w = __shfl(w_mine, j, 64);
+        L += attn_sink_term(a, h, M);
 #pragma unroll
-            for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
-                int d = lane + 64 * i;
-                if (d < hd) o[i] = fmaf(pp[(size_t)(base + j) * stride + 2 + d], w, o[i]);
-            }
-        }
+        for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) o[map][i] /= L;
     }
+    combine_maps<MAPS>(o, a);
     T* orow = out + (size_t)t * a.out_stride + (size_t)h * hd;
-    L += attn_sink_term(a, h, M);
 #pragma unroll
     for (int i = 0; i < MAX_HEAD_DIM / 64; ++i) {
         int d = lane + 64 * i;
-        if (d < hd) orow[d] = from_f32<T>(o[i] / L * attn_gate(a, t, h, d));
+        if (d < hd) orow[d] = from_f32<T>(o[0][i] * attn_gate(a, t, h, d));
     }
 }
 
@@ -388,15 +423,17 @@ static int launch_generic(hipStream_t stream, const T* q, T* out, const T* k_cac
                           const int* block_table, const int* token_entry, const int* positions, const int* q_starts,
                           const int* seq_lens, int n_entries, float* scratch, size_t scratch_bytes, int max_seq_len,
                           int n_single, const AttnArgs& a, int allow_mfma) {
-    bool vec = a.head_dim % 4 == 0 && (uintptr_t)k_cache % (4 * sizeof(T)) == 0;
+    const int map_dim = a.head_dim / a.maps;
+    bool vec = a.head_dim % 4 == 0 && map_dim % 4 == 0 && (uintptr_t)k_cache % (4 * sizeof(T)) == 0;
     // Single-token entries are split by key range when the caller gave room for the partial results.
-    int max_chunks = max_seq_len > 0 ? ceil_div(max_seq_len, GENERIC_CHUNK) : 0;
-    size_t need = (size_t)n_entries * a.n_heads * max_chunks * (a.v_dim + 2) * sizeof(float);
+    int max_chunks = max_seq_len > 0 ? attn_chunks_seen(a, ceil_div(max_seq_len, GENERIC_CHUNK), GENERIC_CHUNK) : 0;
+    const int columns = a.n_heads * a.maps;
+    size_t need = (size_t)n_entries * columns * max_chunks * (a.v_dim + 2) * sizeof(float);
     bool split = max_chunks > 0 && scratch != nullptr && q_starts != nullptr && seq_lens != nullptr &&
-                 scratch_bytes >= need && n_single != 0 && n_entries <= 65535 && max_chunks <= 65535;
+                 scratch_bytes >= need && n_single != 0 && n_entries <= 65535 && max_chunks <= 65535 && columns <= 65535;
     bool only_single = split && n_single == n_entries && a.n_tokens == n_entries;     // every entry brings one token: the caller says so
     const int G = a.n_heads / a.n_kv_heads;
-    const bool groupable = a.head_dim <= GROUP_MAX_HEAD_DIM && a.v_dim <= GROUP_MAX_HEAD_DIM && (G == 2 || G == 4 || G == 8);
+    const bool groupable = a.head_dim <= GROUP_MAX_HEAD_DIM && a.v_dim <= GROUP_MAX_HEAD_DIM && (G == 2 || G == 4 || G == 8) && a.maps == 1;
     bool tiles_took = false;
     if constexpr (std::is_same<T, float>::value) {
         // 32-bit: entries with several tokens go to the matrix cores where the shape allows
@@ -418,12 +455,10 @@ static int launch_generic(hipStream_t stream, const T* q, T* out, const T* k_cac
 #undef TOKENS
         } else {
             dim3 grid(a.n_tokens, a.n_heads);
-            if (vec)
-                attention_generic_kernel<T, true><<<grid, 64, 0, stream>>>(q, out, k_cache, v_cache, block_table, token_entry,
-                                                                        positions, q_starts, split, a);
-            else
-                attention_generic_kernel<T, false><<<grid, 64, 0, stream>>>(q, out, k_cache, v_cache, block_table, token_entry,
-                                                                         positions, q_starts, split, a);
+#define ROWS(V, MM) attention_generic_kernel<T, V, MM><<<grid, 64, 0, stream>>>(q, out, k_cache, v_cache, block_table, token_entry, positions, q_starts, split, a)
+            if (a.maps == 2) { if (vec) ROWS(true, 2); else ROWS(false, 2); }
+            else { if (vec) ROWS(true, 1); else ROWS(false, 1); }
+#undef ROWS
         }
     }
     if (split) {
@@ -451,16 +486,15 @@ static int launch_generic(hipStream_t stream, const T* q, T* out, const T* k_cac
             else { if (vec) GROUP(true, 2); else GROUP(false, 2); }
 #undef GROUP
         } else {
-            dim3 grid(n_entries, a.n_heads, max_chunks);
-            if (vec)
-                attention_generic_split_kernel<T, true><<<grid, 64, 0, stream>>>(q, scratch, k_cache, v_cache, block_table,
-                                                                              q_starts, seq_lens, max_chunks, a);
-            else
-                attention_generic_split_kernel<T, false><<<grid, 64, 0, stream>>>(q, scratch, k_cache, v_cache, block_table,
-                                                                               q_starts, seq_lens, max_chunks, a);
+            dim3 grid(n_entries, columns, max_chunks);
+#define SPLIT(V, MM) attention_generic_split_kernel<T, V, MM><<<grid, 64, 0, stream>>>(q, scratch, k_cache, v_cache, block_table, q_starts, seq_lens, max_chunks, a)
+            if (a.maps == 2) { if (vec) SPLIT(true, 2); else SPLIT(false, 2); }
+            else { if (vec) SPLIT(true, 1); else SPLIT(false, 1); }
+#undef SPLIT
         }
-        attention_generic_merge_kernel<T><<<dim3(n_entries, a.n_heads), 64, 0, stream>>>(scratch, out, q_starts, seq_lens,
-                                                                                        max_chunks, a);
+        dim3 heads(n_entries, a.n_heads);
+        if (a.maps == 2) attention_generic_merge_kernel<T, 2><<<heads, 64, 0, stream>>>(scratch, out, q_starts, seq_lens, max_chunks, a);
+        else attention_generic_merge_kernel<T, 1><<<heads, 64, 0, stream>>>(scratch, out, q_starts, seq_lens, max_chunks, a);
     }
     return 0;
 }
@@ -480,6 +514,9 @@ static int launch_generic(hipStream_t stream, const T* q, T* out, const T* k_cac
 // softcap, keep_first: the soft cap of the scores and the first keys that a window keeps (AttnArgs), or 0.
 // sink: [n_heads] 32-bit, a number a head that the softmax's denominator also holds the exponential of, or null.
 // gate: [n_tokens, gate_stride] 32-bit, one number for every gate_per output features, whose sigmoid they are multiplied by, or null.
+// mask_chunk: > 0: a query sees its own chunk of so many positions only (window 0 then).
+// maps 2: differential attention (AttnArgs): head_dim is the width of a head's row of q and of a key's row, two maps of
+// head_dim / 2 features; diff_lambda, diff_eps, diff_scale as there.  maps 1: they are not used.
 extern "C" int llmrs_attention_ext(hipStream_t stream, int dtype, const void* q, int q_stride, void* out, int out_stride,
                                    const void* k_cache, const void* v_cache, const int* block_table, int table_width,
                                    const int* token_entry, const int* positions, const int* q_starts,
@@ -487,7 +524,8 @@ extern "C" int llmrs_attention_ext(hipStream_t stream, int dtype, const void* q,
                                    int head_dim, int page_size, int num_pages, int window, float scale,
                                    void* scratch, size_t scratch_bytes, int max_seq_len, int n_single, long single_keys,
                                    int allow_mfma, int v_dim, const float* dist_r1, const float* dist_r2, float softcap,
-                                   int keep_first, const float* sink, const float* gate, int gate_stride, int gate_per) {
+                                   int keep_first, const float* sink, const float* gate, int gate_stride, int gate_per, int mask_chunk,
+                                   int maps, float diff_lambda, float diff_eps, float diff_scale) {
     LLMRS_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && head_dim > 0 && v_dim > 0, "attention: bad sizes");
     LLMRS_REQUIRE(v_dim <= MAX_HEAD_DIM, "attention: value width %d exceeds %d", v_dim, MAX_HEAD_DIM);
     LLMRS_REQUIRE((dist_r1 == nullptr) == (dist_r2 == nullptr), "attention: the distance penalty needs both of its tables");
@@ -498,6 +536,9 @@ extern "C" int llmrs_attention_ext(hipStream_t stream, int dtype, const void* q,
     LLMRS_REQUIRE(window >= 0, "attention: negative window");
     LLMRS_REQUIRE(softcap >= 0.0f && keep_first >= 0, "attention: negative soft cap or number of kept first keys");
     LLMRS_REQUIRE(n_heads <= 65535, "attention: too many heads for one launch");
+    LLMRS_REQUIRE(mask_chunk >= 0 && (mask_chunk == 0 || window == 0), "attention: a mask in chunks and a window exclude each other");
+    LLMRS_REQUIRE(maps == 1 || (maps == 2 && head_dim % 2 == 0), "attention: a head has one map, or two of equal width");
+    LLMRS_REQUIRE(maps == 1 || diff_eps > 0.0f, "attention: the norm of the maps' difference needs a positive eps");
     LLMRS_REQUIRE(gate == nullptr || (gate_per > 0 && (n_heads * v_dim) % gate_per == 0 && gate_stride >= n_heads * v_dim / gate_per),
                   "attention: a gate for every %d of %d output features at rows of %d does not fit", gate_per, n_heads * v_dim, gate_stride);
     LLMRS_REQUIRE(n_single <= n_entries, "attention: %d single-token entries among %d entries", n_single, n_entries);
@@ -505,7 +546,7 @@ extern "C" int llmrs_attention_ext(hipStream_t stream, int dtype, const void* q,
                   "attention: every entry is said to bring one token, but %d entries bring %d tokens", n_entries, n_tokens);
     if (n_tokens == 0) return 0;
     AttnArgs a{n_tokens, n_heads, n_kv_heads, head_dim, page_size, table_width, num_pages, q_stride, out_stride, window, scale,
-               v_dim, dist_r1, dist_r2, softcap, window > 0 ? keep_first : 0, sink, gate, gate_stride, gate_per};
+               v_dim, dist_r1, dist_r2, softcap, window > 0 ? keep_first : 0, sink, gate, gate_stride, gate_per, mask_chunk, maps, diff_lambda, diff_eps, diff_scale};
     if (dtype == LLMRS_BF16 && allow_mfma) {
         int took = llmrs_attention_bf16_mfma(stream, (const bf16*)q, (bf16*)out, (const bf16*)k_cache, (const bf16*)v_cache,
                                              block_table, token_entry, positions, q_starts, seq_lens, n_entries,
@@ -538,5 +579,5 @@ extern "C" int llmrs_attention(hipStream_t stream, int dtype, const void* q, int
     return llmrs_attention_ext(stream, dtype, q, q_stride, out, out_stride, k_cache, v_cache, block_table, table_width,
                                token_entry, positions, q_starts, seq_lens, n_entries, n_tokens, n_heads, n_kv_heads,
                                head_dim, page_size, num_pages, window, scale, scratch, scratch_bytes, max_seq_len, n_single,
-                               single_keys, allow_mfma, head_dim, nullptr, nullptr, 0.0f, 0, nullptr, nullptr, 0, 1);
+                               single_keys, allow_mfma, head_dim, nullptr, nullptr, 0.0f, 0, nullptr, nullptr, 0, 1, 0, 1, 0.0f, 0.0f, 0.0f);
 }

@@ -22,10 +22,18 @@ __device__ __forceinline__ bool rows_by_eights(const T* table, const float* out,
 // out[t, :] = float(table[tokens[t], :]) * scale   (reference: embed_batch_*, shaders/ops.metal:878-915,
 // which has no scale: 1 there and for every architecture that does not ask for one)
 // ADD: out[t, :] += the same, in 32-bit (a stream that is shown its tokens' embeddings again).
-template <class T, bool ADD>
+// WAVES: a vector of the token's position is added, feature 2i the sine and 2i + 1 the cosine of positions[t] * rates[i],
+// angle, sine and cosine in 32-bit.
+__device__ __forceinline__ float position_wave(float pos, const float* __restrict__ rates, int d) {
+    float a = pos * rates[d >> 1];
+    return (d & 1) ? cosf(a) : sinf(a);
+}
+template <class T, bool ADD, bool WAVES>
 __global__ void embed_rows_kernel(float* __restrict__ out, const T* __restrict__ table,
-                                  const int* __restrict__ tokens, int D, int V, float scale) {
+                                  const int* __restrict__ tokens, int D, int V, float scale,
+                                  const int* __restrict__ positions, const float* __restrict__ rates) {
     int t = blockIdx.x;
+    const float pos = WAVES ? (float)positions[t] : 0.0f;
     int row = tokens[t];
     row = row < 0 ? 0 : (row >= V ? V - 1 : row);  // the host has checked ids; never read outside the table
     const T* src = table + (size_t)row * D;
@@ -40,12 +48,25 @@ __global__ void embed_rows_kernel(float* __restrict__ out, const T* __restrict__
 #pragma unroll
                     for (int j = 0; j < 4; ++j) { v[j] += a[j]; v[4 + j] += b[j]; }
                 }
+                if constexpr (WAVES) {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        float s, c;
+                        sincosf(pos * rates[(d >> 1) + j], &s, &c);
+                        v[2 * j] += s;
+                        v[2 * j + 1] += c;
+                    }
+                }
                 store8(dst + d, v);
             }
             return;
         }
     }
-    for (int d = threadIdx.x; d < D; d += blockDim.x) dst[d] = (ADD ? dst[d] : 0.0f) + to_f32(src[d]) * scale;
+    for (int d = threadIdx.x; d < D; d += blockDim.x) {
+        float v = (ADD ? dst[d] : 0.0f) + to_f32(src[d]) * scale;
+        if constexpr (WAVES) v += position_wave(pos, rates, d);
+        dst[d] = v;
+    }
 }
 
 // One block per row: ss = sum x^2 in 32-bit, inv = 1/sqrt(ss/D + eps),
@@ -127,14 +148,15 @@ __global__ void rmsnorm_rows_reg_kernel(T* __restrict__ out, const float* __rest
     }
 }
 
-template <bool ADD>
-static int embed_rows(hipStream_t stream, int dtype, float* out, const void* table, const int* tokens, int n_tokens, int D, int V, float scale) {
+template <bool ADD, bool WAVES>
+static int embed_rows(hipStream_t stream, int dtype, float* out, const void* table, const int* tokens, int n_tokens, int D, int V, float scale,
+                      const int* positions = nullptr, const float* rates = nullptr) {
     LLMRS_REQUIRE(n_tokens >= 0 && D > 0 && V > 0, "embed_rows: bad sizes T=%d D=%d V=%d", n_tokens, D, V);
     if (n_tokens == 0) return 0;
     if (dtype == LLMRS_F32)
-        embed_rows_kernel<float, ADD><<<n_tokens, 256, 0, stream>>>(out, (const float*)table, tokens, D, V, scale);
+        embed_rows_kernel<float, ADD, WAVES><<<n_tokens, 256, 0, stream>>>(out, (const float*)table, tokens, D, V, scale, positions, rates);
     else if (dtype == LLMRS_BF16)
-        embed_rows_kernel<bf16, ADD><<<n_tokens, 256, 0, stream>>>(out, (const bf16*)table, tokens, D, V, scale);
+        embed_rows_kernel<bf16, ADD, WAVES><<<n_tokens, 256, 0, stream>>>(out, (const bf16*)table, tokens, D, V, scale, positions, rates);
     else
         return llmrs_fail("embed_rows: unknown dtype %d", dtype);
     LLMRS_LAUNCH_CHECK("embed_rows");
@@ -142,12 +164,113 @@ static int embed_rows(hipStream_t stream, int dtype, float* out, const void* tab
 }
 extern "C" int llmrs_embed_rows(hipStream_t stream, int dtype, float* out, const void* table, const int* tokens,
                                 int n_tokens, int D, int V, float scale) {
-    return embed_rows<false>(stream, dtype, out, table, tokens, n_tokens, D, V, scale);
+    return embed_rows<false, false>(stream, dtype, out, table, tokens, n_tokens, D, V, scale);
 }
 // out[t, :] += float(table[tokens[t], :]) * scale
 extern "C" int llmrs_embed_rows_add(hipStream_t stream, int dtype, float* out, const void* table, const int* tokens,
                                     int n_tokens, int D, int V, float scale) {
-    return embed_rows<true>(stream, dtype, out, table, tokens, n_tokens, D, V, scale);
+    return embed_rows<true, false>(stream, dtype, out, table, tokens, n_tokens, D, V, scale);
+}
+
+// out[t, :] = float(table[tokens[t], :]) * scale + waves of positions[t] (see the kernel); rates: [(D + 1) / 2] 32-bit
+extern "C" int llmrs_embed_rows_waves(hipStream_t stream, int dtype, float* out, const void* table, const int* tokens,
+                                      int n_tokens, int D, int V, float scale, const int* positions, const float* rates) {
+    LLMRS_REQUIRE(positions && rates, "embed_rows: the position vector needs positions and rates");
+    return embed_rows<false, true>(stream, dtype, out, table, tokens, n_tokens, D, V, scale, positions, rates);
+}
+
+// The norm of a sublayer's result on its way into the stream, for sublayers that read the stream as it is: one block a row,
+//   h[t, :] += y[t, :] / sqrt(mean(y^2) + eps) * w      (32-bit)
+//   x[t, :] = the new h[t, :] in the activation type     (x null: not wanted; a 32-bit engine reads h itself)
+//   y[t, :] = 0                                          (where the next sublayer will add its result)
+// norm 0: h stays, only x and y are made (in front of the first sublayer).  HELD: the row in registers between the sum and
+// the stores, four features a piece, everything asked for at once; HELD 0: any width, one feature at a time.
+template <class T, int HELD>
+__global__ __launch_bounds__(256) void post_norm_rows_kernel(float* __restrict__ h, float* __restrict__ y, const float* __restrict__ w,
+                                                             T* __restrict__ x, int D, float eps, int norm) {
+    __shared__ float partial[4];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    float* hrow = h + (size_t)blockIdx.x * D;
+    float* yrow = y + (size_t)blockIdx.x * D;
+    T* xrow = x ? x + (size_t)blockIdx.x * D : nullptr;
+    if constexpr (HELD > 0) {
+        const int n4 = D / 4;
+        const f32x4 none = {0.f, 0.f, 0.f, 0.f};
+        f32x4 yv[HELD], hv[HELD], wv[HELD];
+        float ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < HELD; ++i) {
+            int idx = i * 256 + threadIdx.x;
+            bool in = idx < n4;
+            yv[i] = in && norm ? ((const f32x4*)yrow)[idx] : none;
+            hv[i] = in ? ((const f32x4*)hrow)[idx] : none;
+            wv[i] = in && norm ? ((const f32x4*)w)[idx] : none;
+        }
+        float inv = 0.0f;
+        if (norm) {                                   // (the same in all threads)
+#pragma unroll
+            for (int i = 0; i < HELD; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) ss = fmaf(yv[i][j], yv[i][j], ss);
+            ss = wave_sum(ss);
+            if (lane == 0) partial[wave] = ss;
+            __syncthreads();
+            inv = 1.0f / sqrtf((partial[0] + partial[1] + partial[2] + partial[3]) / (float)D + eps);
+        }
+#pragma unroll
+        for (int i = 0; i < HELD; ++i) {
+            int idx = i * 256 + threadIdx.x;
+            if (idx >= n4) continue;
+            f32x4 v;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = hv[i][j] + yv[i][j] * inv * wv[i][j];
+            if (norm) ((f32x4*)hrow)[idx] = v;
+            ((f32x4*)yrow)[idx] = none;
+            if (xrow) {
+                typedef T T4 __attribute__((ext_vector_type(4)));
+                T4 o;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) o[j] = from_f32<T>(v[j]);
+                *(T4*)(xrow + idx * 4) = o;
+            }
+        }
+    } else {
+        float inv = 0.0f;
+        if (norm) {
+            float ss = 0.0f;
+            for (int d = threadIdx.x; d < D; d += 256) ss = fmaf(yrow[d], yrow[d], ss);
+            ss = wave_sum(ss);
+            if (lane == 0) partial[wave] = ss;
+            __syncthreads();
+            inv = 1.0f / sqrtf((partial[0] + partial[1] + partial[2] + partial[3]) / (float)D + eps);
+        }
+        for (int d = threadIdx.x; d < D; d += 256) {
+            float v = hrow[d];
+            if (norm) {
+                v += yrow[d] * inv * w[d];
+                hrow[d] = v;
+            }
+            yrow[d] = 0.0f;
+            if (xrow) xrow[d] = from_f32<T>(v);
+        }
+    }
+}
+
+// weight null: no norm (norm 0 above); x null or in `dtype`.
+extern "C" int llmrs_post_norm_rows(hipStream_t stream, int dtype, float* h, float* y, const float* weight, void* x, int n_rows, int D, float eps) {
+    LLMRS_REQUIRE(h && y && n_rows >= 0 && D > 0, "post_norm: bad sizes rows=%d D=%d", n_rows, D);
+    LLMRS_REQUIRE(!weight || eps > 0.0f, "post_norm: eps must be positive, got %g", eps);
+    if (n_rows == 0) return 0;
+    if (dtype != LLMRS_F32 && dtype != LLMRS_BF16) return llmrs_fail("post_norm: unknown dtype %d", dtype);
+    bool pieces = D % 4 == 0 && D <= 4 * 256 * 8 && ((uintptr_t)h & 15) == 0 && ((uintptr_t)y & 15) == 0 && ((uintptr_t)weight & 15) == 0 && ((uintptr_t)x & 15) == 0;
+    int held = !pieces ? 0 : D <= 4 * 256 ? 1 : D <= 4 * 256 * 2 ? 2 : D <= 4 * 256 * 4 ? 4 : 8;
+#define POST(T, N) post_norm_rows_kernel<T, N><<<n_rows, 256, 0, stream>>>(h, y, weight, (T*)x, D, eps, weight != nullptr)
+#define POST_BY_WIDTH(T) do { if (held == 0) POST(T, 0); else if (held == 1) POST(T, 1); else if (held == 2) POST(T, 2); else if (held == 4) POST(T, 4); else POST(T, 8); } while (0)
+    if (dtype == LLMRS_F32) POST_BY_WIDTH(float); else POST_BY_WIDTH(bf16);
+#undef POST_BY_WIDTH
+#undef POST
+    LLMRS_LAUNCH_CHECK("post_norm");
+    return 0;
 }
 
 // rows == nullptr: row i of x -> row i of out; else row rows[i] of x -> row i of out.

@@ -9,12 +9,16 @@
 //   rot: features (2i, 2i + 1), i < rotary_dim / 2, turned by the angle position * inv_freq[i], cosine and sine both
 //        times `gain`; the others pass
 //   k likewise (weight w_k), into its page; v[t, g, :] = u_v + bias_v, into its page (values lie transposed, cache_layout.h).
+// With `maps` = 2 a head of q or k is two such heads of head_dim features one after the other (the two maps of differential
+// attention): each is normed and turned by itself, and the two halves of a key lie side by side in one row of the cache,
+// 2 head_dim wide; values have one head for both.
 // Everything is computed in 32-bit and rounded once to the activation type on the way out.
 #include "cache_layout.h"
 #include "common.h"
 
 struct QkvFinishArgs {
-    int n_tokens, n_heads, n_kv_heads, head_dim, v_dim;
+    int n_tokens, n_heads, n_kv_heads, head_dim, v_dim;    // n_heads, n_kv_heads: times `maps` where q and k are meant (q_heads, k_heads)
+    int maps;
     int in_stride, q_stride;       // elements between tokens in the sums and in q
     int page_size, num_pages, write_kv;
     float eps;                     // of the unit norm; 0: q and k are not normed
@@ -30,7 +34,13 @@ struct QkvFinishArgs {
     const int* q_starts;
     const int* slots;
     const int* token_entry;
+    __host__ __device__ int q_heads() const { return n_heads * maps; }
+    __host__ __device__ int k_heads() const { return n_kv_heads * maps; }
 };
+// Where feature d of k head `head` (counted over maps) lies: both maps of a key side by side in its row.
+__device__ __forceinline__ size_t finished_key_index(const QkvFinishArgs& a, int page, int head, int off, int d) {
+    return k_cache_index(page, head / a.maps, off, (head % a.maps) * a.head_dim + d, a.n_kv_heads, a.page_size, a.maps * a.head_dim);
+}
 
 // One wave for each (token, head of q, k or v); a block's four waves take four neighbouring tokens of the same head
 // (a quarter of the blocks to hand out, and the rows that a convolution reads again lie in the same block's reach).
@@ -43,12 +53,13 @@ __global__ __launch_bounds__(256) void qkv_finish_kernel(const float* __restrict
                                                          QkvFinishArgs a) {
     int t = blockIdx.x * 4 + (threadIdx.x >> 6), head = blockIdx.y, lane = threadIdx.x & 63;
     if (t >= a.n_tokens) return;
-    bool is_q = head < a.n_heads, is_k = !is_q && head < a.n_heads + a.n_kv_heads;
+    const int qh = a.q_heads(), qkh = qh + a.k_heads();
+    bool is_q = head < qh, is_k = !is_q && head < qkh;
     if (!is_q && !a.write_kv) return;
     int width = (is_q || is_k) ? a.head_dim : a.v_dim;
     int col = is_q ? head * a.head_dim
-                   : is_k ? a.n_heads * a.head_dim + (head - a.n_heads) * a.head_dim
-                          : (a.n_heads + a.n_kv_heads) * a.head_dim + (head - a.n_heads - a.n_kv_heads) * a.v_dim;
+                   : is_k ? head * a.head_dim
+                          : qkh * a.head_dim + (head - qkh) * a.v_dim;
     const float* src = sums + (size_t)t * a.in_stride + col;
     float x[NI];           // features lane, lane + 64, ... (heads of up to 512)
     float ss = 0.0f;
@@ -138,9 +149,9 @@ __global__ __launch_bounds__(256) void qkv_finish_kernel(const float* __restrict
         int d = lane + 64 * i;
         if (d >= width) continue;
         if (is_k)
-            k_cache[k_cache_index(page, head - a.n_heads, off, d, a.n_kv_heads, a.page_size, a.head_dim)] = from_f32<T>(x[i] * inv);
+            k_cache[finished_key_index(a, page, head - qh, off, d)] = from_f32<T>(x[i] * inv);
         else
-            v_cache[v_cache_index(page, head - a.n_heads - a.n_kv_heads, off, d, a.n_kv_heads, a.page_size, a.v_dim)] = from_f32<T>(x[i]);
+            v_cache[v_cache_index(page, head - qkh, off, d, a.n_kv_heads, a.page_size, a.v_dim)] = from_f32<T>(x[i]);
     }
 }
 
@@ -176,7 +187,7 @@ __global__ __launch_bounds__(256) void qkv_finish_wide_kernel(const float* __res
     constexpr int QKV_WIDE_TOKENS = 4 * TPW;
     const int t0 = blockIdx.x * QKV_WIDE_TOKENS;
     const int c = blockIdx.y * 256 + 4 * lane;                 // this lane's first column
-    const int q_cols = a.n_heads * a.head_dim, qk_cols = q_cols + a.n_kv_heads * a.head_dim;
+    const int q_cols = a.q_heads() * a.head_dim, qk_cols = q_cols + a.k_heads() * a.head_dim;
     const bool inside = c < a.columns, is_q = c < q_cols, is_k = !is_q && c < qk_cols, is_v = inside && !is_q && !is_k;
     const bool works = inside && (is_q || a.write_kv);
     const int d = (is_q || is_k) ? c % a.head_dim : 0;          // the first of the lane's four features within its head
@@ -292,7 +303,7 @@ __global__ __launch_bounds__(256) void qkv_finish_wide_kernel(const float* __res
         int page = slot / a.page_size, off = slot % a.page_size;
         if (is_k) {
             int head = (c - q_cols) / a.head_dim;
-            qkv_store4<T>(k_cache + k_cache_index(page, head, off, d, a.n_kv_heads, a.page_size, a.head_dim), x);
+            qkv_store4<T>(k_cache + finished_key_index(a, page, head, off, d), x);
         } else if (is_v) {
             int idx = c - qk_cols, head = idx / a.v_dim, dv = idx % a.v_dim;
 #pragma unroll
@@ -308,31 +319,33 @@ __global__ __launch_bounds__(256) void qkv_finish_wide_kernel(const float* __res
 // positions: [n_tokens], inv_freq: [rotary_dim / 2] 32-bit, for the rotation (rotary_dim 0: none); gain: see above.
 // q_weight, k_weight: [head_dim] 32-bit or null.  taps: [columns of q | k | v][n_taps] 32-bit or null; then state (null when
 // n_taps == 1), q_starts [n_entries + 1], slots [n_entries], token_entry [n_tokens] say where a token's earlier rows lie.
+// maps: 1, or 2: every head of q and k is two heads of head_dim features (see above).
 // The state is only read here: llmrs_conv_state_update brings it up to date afterwards.
 extern "C" int llmrs_qkv_finish(hipStream_t stream, int dtype, const float* sums, int in_stride, const float* bias, void* q,
                                 int q_stride, const int* slot_map, void* k_cache, void* v_cache, int n_tokens, int n_heads,
                                 int n_kv_heads, int head_dim, int v_dim, int page_size, int num_pages, int write_kv, float eps,
                                 const int* positions, const float* inv_freq, int rotary_dim, const float* q_weight,
                                 const float* k_weight, float gain, const float* taps, int n_taps, const float* state,
-                                long state_stride, const int* q_starts, const int* slots, const int* token_entry, int n_entries) {
+                                long state_stride, const int* q_starts, const int* slots, const int* token_entry, int n_entries, int maps) {
     LLMRS_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads >= 0 && head_dim > 0 && v_dim > 0, "qkv_finish: bad sizes");
     LLMRS_REQUIRE(head_dim <= 512 && v_dim <= 512, "qkv_finish: heads of %d / %d features exceed 512", head_dim, v_dim);
-    LLMRS_REQUIRE(in_stride >= (n_heads + n_kv_heads) * head_dim + n_kv_heads * v_dim && q_stride >= n_heads * head_dim,
+    LLMRS_REQUIRE(maps == 1 || maps == 2, "qkv_finish: a head has one or two maps, not %d", maps);
+    LLMRS_REQUIRE(in_stride >= (n_heads + n_kv_heads) * maps * head_dim + n_kv_heads * v_dim && q_stride >= n_heads * maps * head_dim,
                   "qkv_finish: row stride too short");
     LLMRS_REQUIRE(eps >= 0.0f, "qkv_finish: negative eps");
     LLMRS_REQUIRE(rotary_dim >= 0 && rotary_dim % 2 == 0 && rotary_dim <= head_dim, "qkv_finish: a rotation of %d features does not fit heads of %d", rotary_dim, head_dim);
     LLMRS_REQUIRE(rotary_dim == 0 || (positions && inv_freq), "qkv_finish: a rotation needs positions and frequencies");
     LLMRS_REQUIRE(!write_kv || (page_size > 0 && num_pages > 0 && slot_map && k_cache && v_cache), "qkv_finish: no cache to write");
-    LLMRS_REQUIRE(n_heads + 2 * n_kv_heads <= 65535, "qkv_finish: too many heads for one launch");
+    LLMRS_REQUIRE((n_heads + n_kv_heads) * maps + n_kv_heads <= 65535, "qkv_finish: too many heads for one launch");
     LLMRS_REQUIRE((q_weight == nullptr && k_weight == nullptr) || eps > 0.0f, "qkv_finish: a norm's weight without the norm");
-    int columns = (n_heads + n_kv_heads) * head_dim + n_kv_heads * v_dim;
+    int columns = (n_heads + n_kv_heads) * maps * head_dim + n_kv_heads * v_dim;
     if (taps) {
         LLMRS_REQUIRE(n_taps >= 1 && bias == nullptr, "qkv_finish: a convolution needs at least one tap and goes without biases");
         LLMRS_REQUIRE(q_starts && slots && token_entry && n_entries > 0, "qkv_finish: a convolution needs the step's entries");
         LLMRS_REQUIRE(n_taps == 1 || (state && state_stride >= (long)(n_taps - 1) * columns), "qkv_finish: the convolution's state is too small");
     }
     if (n_tokens == 0) return 0;
-    QkvFinishArgs a{n_tokens, n_heads, n_kv_heads, head_dim, v_dim, in_stride, q_stride, page_size, num_pages, write_kv, eps, rotary_dim,
+    QkvFinishArgs a{n_tokens, n_heads, n_kv_heads, head_dim, v_dim, maps, in_stride, q_stride, page_size, num_pages, write_kv, eps, rotary_dim,
                     gain, q_weight, k_weight, taps, n_taps, columns, state, state_stride, q_starts, slots, token_entry};
     // four columns a lane where the heads and the rows allow it
     auto pieces = [](const void* p) { return p == nullptr || ((uintptr_t)p & 15) == 0; };
@@ -352,7 +365,7 @@ extern "C" int llmrs_qkv_finish(hipStream_t stream, int dtype, const float* sums
         LLMRS_LAUNCH_CHECK("qkv_finish");
         return 0;
     }
-    dim3 grid(ceil_div(n_tokens, 4), n_heads + 2 * n_kv_heads);
+    dim3 grid(ceil_div(n_tokens, 4), (n_heads + n_kv_heads) * maps + n_kv_heads);
     int widest = head_dim > v_dim ? head_dim : v_dim;
     if (dtype != LLMRS_F32 && dtype != LLMRS_BF16) return llmrs_fail("qkv_finish: unknown dtype %d", dtype);
 #define QKV_FINISH(T, NI) qkv_finish_kernel<T, NI><<<grid, 256, 0, stream>>>(sums, bias, (T*)q, slot_map, (T*)k_cache, (T*)v_cache, positions, inv_freq, a)

@@ -4,7 +4,9 @@
 // The router: scores = softmax over all experts of the 32-bit logits; the `top` largest are chosen (of equal scores the
 // lower index first); an expert's weight is its score, as it is or divided by the chosen scores' sum.  Or (score kind
 // 1) scores = sigmoid(logit) for each expert by itself, chosen by score + correction[e], weighed by the score without
-// it (divided by the chosen scores' sum + 1e-20 with `renormalize`), times `scale`.  The experts' up
+// it (divided by the chosen scores' sum + 1e-20 with `renormalize`), times `scale`.  With `groups` > 1 the experts form so
+// many equal groups of neighbours, and only those of the `keep_groups` best groups can be chosen, a group being as good as
+// its best expert (by what the choice goes by; of equal groups the lower index first).  The experts' up
 // matrices lie one under the other and their down matrices side by side, so that the experts of a token are a dense
 // feed-forward of experts * ff hidden units whose activations are multiplied by the expert's weight, zero for the
 // experts that were not chosen: the activation kernel below applies act and that weight in one pass.
@@ -12,11 +14,55 @@
 
 #define ROUTE_MAX_EXPERTS 1024
 
-// One wave a token.  weights [T, E] 32-bit: the chosen experts' weights, zero elsewhere.
+// The best of a wave's lanes: the largest value, of equal values the lowest index.
+__device__ __forceinline__ void wave_best(float& best, int& at) {
+#pragma unroll
+    for (int d = 32; d > 0; d >>= 1) {
+        float ob = __shfl_xor(best, d, 64);
+        int oa = __shfl_xor(at, d, 64);
+        if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+    }
+}
+
+// Takes the experts outside the `keep` best of `groups` groups out of the choice: c[i] (what the choice of expert lane +
+// 64 i goes by) becomes `gone` there.  room: 2 ROUTE_MAX_EXPERTS floats of LDS.  All lanes of the block's one wave.
+template <int PER>
+__device__ __forceinline__ void keep_best_groups(float (&c)[PER], int E, int groups, int keep, float gone, float* room) {
+    const int lane = threadIdx.x, per = E / groups;
+    float* choice = room;
+    float* group = room + ROUTE_MAX_EXPERTS;          // a group's score; once it is kept, what no score is
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+        if (lane + 64 * i < E) choice[lane + 64 * i] = c[i];
+    __syncthreads();
+    for (int g = lane; g < groups; g += 64) {
+        float best = choice[g * per];
+        for (int j = 1; j < per; ++j) best = fmaxf(best, choice[g * per + j]);
+        group[g] = best;
+    }
+    __syncthreads();
+    for (int r = 0; r < keep; ++r) {
+        float best = -INFINITY;
+        int at = 0x7fffffff;
+        for (int g = lane; g < groups; g += 64)
+            if (group[g] < INFINITY && group[g] > best) { best = group[g]; at = g; }
+        wave_best(best, at);
+        if (at < groups && (at & 63) == lane) group[at] = INFINITY;
+        __syncthreads();
+    }
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        int e = lane + 64 * i;
+        if (e < E && group[e / per] < INFINITY) c[i] = gone;
+    }
+}
+
+// One wave a token; a lane holds PER experts (E <= 64 PER).  weights [T, E] 32-bit: the chosen experts' weights, zero elsewhere.
+template <int PER>
 __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict__ logits, int ld, float* __restrict__ weights, int ldw,
-                                                         int E, int top, int renormalize) {
+                                                         int E, int top, int renormalize, int groups, int keep_groups) {
+    __shared__ float room[2 * ROUTE_MAX_EXPERTS];
     int t = blockIdx.x, lane = threadIdx.x;
-    constexpr int PER = ROUTE_MAX_EXPERTS / 64;
     float z[PER];
     float mx = -INFINITY;
 #pragma unroll
@@ -33,6 +79,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
         sum += fmaxf(z[i], 0.0f);
     }
     float inv = 1.0f / wave_sum(sum);
+    if (groups > 1) keep_best_groups<PER>(z, E, groups, keep_groups, -1.0f, room);
     float keep[PER];
 #pragma unroll
     for (int i = 0; i < PER; ++i) keep[i] = 0.0f;
@@ -43,13 +90,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
 #pragma unroll
         for (int i = 0; i < PER; ++i)
             if (z[i] > best) { best = z[i]; at = lane + 64 * i; }      // ascending index within a lane: the first of equals stays
-        // the wave's best: the largest score, of equal scores the lowest index
-#pragma unroll
-        for (int d = 32; d > 0; d >>= 1) {
-            float ob = __shfl_xor(best, d, 64);
-            int oa = __shfl_xor(at, d, 64);
-            if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
-        }
+        wave_best(best, at);
         if (best < 0.0f) break;
         chosen_sum += best * inv;
 #pragma unroll
@@ -65,11 +106,12 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
 }
 
 // Score kind 1.  One wave a token; the chosen experts' weights into weights [T, E], zero elsewhere.
+template <int PER>
 __global__ __launch_bounds__(64) void route_topk_sigmoid_kernel(const float* __restrict__ logits, int ld, float* __restrict__ weights, int ldw,
                                                                  int E, int top, int renormalize, const float* __restrict__ correction,
-                                                                 float scale) {
+                                                                 float scale, int groups, int keep_groups) {
+    __shared__ float room[2 * ROUTE_MAX_EXPERTS];
     int t = blockIdx.x, lane = threadIdx.x;
-    constexpr int PER = ROUTE_MAX_EXPERTS / 64;
     float s[PER], c[PER], keep[PER];        // score, what the choice goes by (-inf: not there or taken), the weight kept
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
@@ -79,6 +121,7 @@ __global__ __launch_bounds__(64) void route_topk_sigmoid_kernel(const float* __r
         c[i] = in ? s[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
         keep[i] = 0.0f;
     }
+    if (groups > 1) keep_best_groups<PER>(c, E, groups, keep_groups, -INFINITY, room);
     float chosen_sum = 0.0f;
     for (int r = 0; r < top; ++r) {
         float best = -INFINITY, best_s = 0.0f;
@@ -107,16 +150,22 @@ __global__ __launch_bounds__(64) void route_topk_sigmoid_kernel(const float* __r
 }
 
 // score_kind 0: softmax over the experts (correction and scale are not used: null and 1); 1: a sigmoid for each expert,
-// chosen by score + correction [E] (null: none), weights times scale.
+// chosen by score + correction [E] (null: none), weights times scale.  groups, keep_groups: see above (1, 1: no groups).
 extern "C" int llmrs_route_topk(hipStream_t stream, const float* logits, int ld, float* weights, int ldw, int n_tokens, int E, int top,
-                                int renormalize, int score_kind, const float* correction, float scale) {
+                                int renormalize, int score_kind, const float* correction, float scale, int groups, int keep_groups) {
     LLMRS_REQUIRE(logits && weights && E > 0 && top > 0 && top <= E && ld >= E && ldw >= E, "route_topk: bad arguments");
     LLMRS_REQUIRE(E <= ROUTE_MAX_EXPERTS, "route_topk: %d experts exceed %d", E, ROUTE_MAX_EXPERTS);
     LLMRS_REQUIRE(score_kind == 0 || score_kind == 1, "route_topk: unknown score kind %d (0: softmax, 1: sigmoid)", score_kind);
     LLMRS_REQUIRE(score_kind == 1 || (correction == nullptr && scale == 1.0f), "route_topk: a correction or a scale goes with sigmoid scores");
+    LLMRS_REQUIRE(groups >= 1 && E % groups == 0 && keep_groups >= 1 && keep_groups <= groups, "route_topk: %d experts in %d groups of which %d", E, groups, keep_groups);
+    LLMRS_REQUIRE(top <= E / groups * keep_groups, "route_topk: top %d of the %d experts of %d groups", top, E / groups * keep_groups, keep_groups);
     if (n_tokens <= 0) return 0;
-    if (score_kind == 1) route_topk_sigmoid_kernel<<<n_tokens, 64, 0, stream>>>(logits, ld, weights, ldw, E, top, renormalize, correction, scale);
-    else route_topk_kernel<<<n_tokens, 64, 0, stream>>>(logits, ld, weights, ldw, E, top, renormalize);
+#define ROUTE(PER) do { if (score_kind == 1) route_topk_sigmoid_kernel<PER><<<n_tokens, 64, 0, stream>>>(logits, ld, weights, ldw, E, top, renormalize, correction, scale, groups, keep_groups); \
+                        else route_topk_kernel<PER><<<n_tokens, 64, 0, stream>>>(logits, ld, weights, ldw, E, top, renormalize, groups, keep_groups); } while (0)
+    if (E <= 64) ROUTE(1);
+    else if (E <= 256) ROUTE(4);
+    else ROUTE(ROUTE_MAX_EXPERTS / 64);
+#undef ROUTE
     LLMRS_LAUNCH_CHECK("route_topk");
     return 0;
 }
@@ -124,6 +173,7 @@ extern "C" int llmrs_route_topk(hipStream_t stream, const float* logits, int ld,
 // out[t, c] = act * (weights ? weights[t, c / ff] : 1); up 32-bit sums, out in the activation type (one rounding).
 // kind 0: act = relu(up[t, c])^2.  kind 1, a gated activation on sums whose columns are (gate_0, up_0, gate_1, up_1, ...):
 // g = min(up[t, 2c], limit), u = clamp(up[t, 2c + 1], -limit, limit), act = g * sigmoid(alpha * g) * (u + 1).
+// kind 2, gated, columns as for kind 1: act = silu(gate) * up.
 template <class T, int KIND>
 __global__ void act_weight_kernel(const float* __restrict__ up, int ldu, const float* __restrict__ weights, int ldw, int ff, int n,
                                   long total, T* __restrict__ out, int ldo, float limit, float alpha) {
@@ -135,6 +185,9 @@ __global__ void act_weight_kernel(const float* __restrict__ up, int ldu, const f
     if constexpr (KIND == 0) {
         float x = fmaxf(up[(size_t)t * ldu + c], 0.0f);
         y = x * x;
+    } else if constexpr (KIND == 2) {
+        float2 gu = *(const float2*)(up + (size_t)t * ldu + 2 * c);
+        y = silu_f32(gu.x) * gu.y;
     } else {
         float2 gu = *(const float2*)(up + (size_t)t * ldu + 2 * c);
         float g = fminf(gu.x, limit), u = fminf(fmaxf(gu.y, -limit), limit);
@@ -144,21 +197,22 @@ __global__ void act_weight_kernel(const float* __restrict__ up, int ldu, const f
     out[(size_t)t * ldo + c] = from_f32<T>(y);
 }
 
-// n: columns of out; up has n columns (kind 0) or 2 n (kind 1, then ldu even and up 8-byte aligned).
+// n: columns of out; up has n columns (kind 0) or 2 n (kinds 1 and 2, then ldu even and up 8-byte aligned).
 extern "C" int llmrs_act_weight(hipStream_t stream, int dtype, const float* up, int ldu, const float* weights, int ldw, int ff,
                                 int n_tokens, int n, int kind, void* out, int ldo, float limit, float alpha) {
     LLMRS_REQUIRE(up && out && n > 0 && ldo >= n && ff > 0 && n % ff == 0, "act_weight: bad arguments");
-    LLMRS_REQUIRE(kind == 0 || kind == 1, "act_weight: unknown activation %d (0: squared relu, 1: clamped gated sigmoid)", kind);
-    LLMRS_REQUIRE(ldu >= (kind == 1 ? 2 * n : n), "act_weight: the sums' rows are too short");
-    LLMRS_REQUIRE(kind == 0 || (ldu % 2 == 0 && ((uintptr_t)up & 7) == 0 && limit > 0.0f), "act_weight: gate and up side by side in 8-byte pairs, and a positive limit");
+    LLMRS_REQUIRE(kind >= 0 && kind <= 2, "act_weight: unknown activation %d (0: squared relu, 1: clamped gated sigmoid, 2: gated silu)", kind);
+    LLMRS_REQUIRE(ldu >= (kind > 0 ? 2 * n : n), "act_weight: the sums' rows are too short");
+    LLMRS_REQUIRE(kind == 0 || (ldu % 2 == 0 && ((uintptr_t)up & 7) == 0), "act_weight: gate and up side by side in 8-byte pairs");
+    LLMRS_REQUIRE(kind != 1 || limit > 0.0f, "act_weight: a positive limit");
     LLMRS_REQUIRE(!weights || ldw >= n / ff, "act_weight: the weights' rows are too short");
     long total = (long)n_tokens * n;
     if (total <= 0) return 0;
     LLMRS_REQUIRE(ceil_div(total, 256) <= 0x7fffffff, "act_weight: too many elements for one launch");
     int blocks = ceil_div(total, 256);
 #define ACT(TT, KK) act_weight_kernel<TT, KK><<<blocks, 256, 0, stream>>>(up, ldu, weights, ldw, ff, n, total, (TT*)out, ldo, limit, alpha)
-    if (dtype == LLMRS_F32) { if (kind == 0) ACT(float, 0); else ACT(float, 1); }
-    else if (dtype == LLMRS_BF16) { if (kind == 0) ACT(bf16, 0); else ACT(bf16, 1); }
+    if (dtype == LLMRS_F32) { if (kind == 0) ACT(float, 0); else if (kind == 1) ACT(float, 1); else ACT(float, 2); }
+    else if (dtype == LLMRS_BF16) { if (kind == 0) ACT(bf16, 0); else if (kind == 1) ACT(bf16, 1); else ACT(bf16, 2); }
     else return llmrs_fail("act_weight: unknown dtype %d", dtype);
 #undef ACT
     LLMRS_LAUNCH_CHECK("act_weight");

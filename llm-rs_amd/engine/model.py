@@ -31,6 +31,7 @@ class Model:
         self.final_norm = build_norm(spec.final_norm, dtype) if spec.final_norm is not None else None
         self.embedding: Optional[torch.Tensor] = None
         self.head: Optional[torch.Tensor] = None
+        self.wave_rates: Optional[torch.Tensor] = None
         keyed = {}
         for block in self.blocks:
             for part in block.parts():
@@ -62,6 +63,9 @@ class Model:
         self.embedding = place(tensors[s.embedding_name], self.device, self.dtype)
         # tied: the output matrix is the token table (src/arch/llama.rs:81)
         self.head = self.embedding if s.head_name is None else place(tensors[s.head_name], self.device, self.dtype)
+        if s.position_wave_base > 0:
+            i = torch.arange((s.hidden_size + 1) // 2, dtype=torch.float64)
+            self.wave_rates = torch.pow(torch.tensor(s.position_wave_base, dtype=torch.float64), -2.0 * i / s.hidden_size).float().to(self.device)
         for block in self.blocks:
             for part in block.parts():
                 part.load(tensors, self.device)
@@ -121,7 +125,8 @@ class Model:
             k.streams_copy_first(h)
         else:
             h = ctx.workspace("model.h", (T, self.spec.hidden_size), torch.float32)
-            k.embed_rows(h, self.embedding, ctx.tokens, self.spec.embedding_scale)
+            k.embed_rows(h, self.embedding, ctx.tokens, self.spec.embedding_scale,
+                         **({} if self.wave_rates is None else {"waves": (ctx.positions, self.wave_rates)}))
         ctx.note_left(h, None)
         for i, run in enumerate(self.spec.schedule):
             ctx.run_index = i

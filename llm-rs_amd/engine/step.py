@@ -117,12 +117,16 @@ class StepContext:
     def workspace(self, name: str, shape, dtype: torch.dtype) -> torch.Tensor:
         return self._runner.workspace(name, shape, dtype)
 
-    def single_keys(self, window: int = 0) -> int:
-        """How many keys the single-token entries see together, each through a window of `window` keys (0: all)."""
-        got = self._keys_seen.get(window)
+    def single_keys(self, window: int = 0, mask_chunk: int = 0) -> int:
+        """How many keys the single-token entries see together, each through a window of `window` keys (0: all) or in its
+        own chunk of `mask_chunk` positions (0: no chunks)."""
+        got = self._keys_seen.get((window, mask_chunk))
         if got is None:
-            got = sum(self.single_lens) if window <= 0 else sum(min(n, window) for n in self.single_lens)
-            self._keys_seen[window] = got
+            if mask_chunk > 0:
+                got = sum((n - 1) % mask_chunk + 1 for n in self.single_lens)
+            else:
+                got = sum(self.single_lens) if window <= 0 else sum(min(n, window) for n in self.single_lens)
+            self._keys_seen[(window, mask_chunk)] = got
         return got
 
     def room_for_next_norm(self, h: torch.Tensor, w: torch.Tensor):

@@ -62,6 +62,17 @@ class NextNorm:
         return self.eps > 0.0
 
 
+class StreamRows:
+    """What a norm on the way into the stream leaves for the sublayer that reads the stream itself (`Kernels.post_norm`):
+    `y`, the stream's rows in the activation type (the stream's own tensor in a 32-bit engine), not normed, and
+    `room`, cleared 32-bit rows for that sublayer to add its result into."""
+
+    weight, whole, eps = None, False, 0.0       # (of no norm: no norm takes these rows for its own)
+
+    def __init__(self, y: torch.Tensor, room: torch.Tensor):
+        self.y, self.room = y, room
+
+
 class KernelTimes:
     """Per-kernel device time with the bytes each call has to move and the operations it has to
     do, as the reference keeps when LLM_PERF is set (src/backend/metal/mod.rs:321-400): a pair of
@@ -177,6 +188,8 @@ class HipKernels(Kernels):
         sigs = {
             "llmrs_embed_rows": [V, I, V, V, V, I, I, I, F],
             "llmrs_embed_rows_add": [V, I, V, V, V, I, I, I, F],
+            "llmrs_embed_rows_waves": [V, I, V, V, V, I, I, I, F, V, V],
+            "llmrs_post_norm_rows": [V, I, V, V, V, V, I, I, F],
             "llmrs_dyt": [V, I, V, V, V, V, V, V, I, I, V, V, V, V],
             "llmrs_conv_state_update": [V, V, I, V, ctypes.c_long, V, V, I, I, I],
             "llmrs_sigmoid_gate": [V, I, V, I, V, I, I, I, I],
@@ -200,17 +213,17 @@ class HipKernels(Kernels):
             "llmrs_argmax_rows": [V, V, I, I, I, V, V, c_size_t],
             "llmrs_sample_rows": [V, V, I, I, I, V, V],
             "llmrs_place_ids": [V, V, I, V, V, V, I, I, I],
-            "llmrs_attention_ext": [V, I, V, I, V, I, V, V, V, I, V, V, V, V, I, I, I, I, I, I, I, I, F, V, c_size_t, I, I, ctypes.c_long, I, I, V, V, F, I, V, V, I, I],
+            "llmrs_attention_ext": [V, I, V, I, V, I, V, V, V, I, V, V, V, V, I, I, I, I, I, I, I, I, F, V, c_size_t, I, I, ctypes.c_long, I, I, V, V, F, I, V, V, I, I, I, I, F, F, F],
             "llmrs_group_rmsnorm": [V, I, V, V, ctypes.c_long, I, V, V, V, I, I, I, F, V, V, V, V, V],
             "llmrs_streams_mix": [V, V, ctypes.c_long, I, V, V, V, ctypes.c_long],
             "llmrs_streams_copy_first": [V, V, ctypes.c_long, I, ctypes.c_long],
-            "llmrs_qkv_finish": [V, I, V, I, V, V, I, V, V, V, I, I, I, I, I, I, I, I, F, V, V, I, V, V, F, V, I, V, ctypes.c_long, V, V, V, I],
+            "llmrs_qkv_finish": [V, I, V, I, V, V, I, V, V, V, I, I, I, I, I, I, I, I, F, V, V, I, V, V, F, V, I, V, ctypes.c_long, V, V, V, I, I],
             "llmrs_linear_scan": [V, V, I, V, I, V, I, V, I, V, V, I, V, ctypes.c_long, V, V, I, I, I, I, I, I, V, I, V, V, I, I],
             "llmrs_silu_columns": [V, V, I, I, I, I],
             "llmrs_delta_prepare": [V, V, I, V, I, V, I, V, I, V, V, I, I, I, I, F],
             "llmrs_gated_rmsnorm": [V, I, V, I, V, I, V, I, I, I, I, F, V, I, I, V, I, F, F],
             "llmrs_rmsnorm_sum": [V, V, V, V, V, V, V, V, I, I, F, F],
-            "llmrs_route_topk": [V, V, I, V, I, I, I, I, I, I, V, F],
+            "llmrs_route_topk": [V, V, I, V, I, I, I, I, I, I, V, F, I, I],
             "llmrs_act_weight": [V, I, V, I, V, I, I, I, I, I, V, I, F, F],
             "llmrs_add_bias_rows": [V, V, I, V, I, I],
             "llmrs_route_counts": [V, V, I, I, I, V],
@@ -310,9 +323,17 @@ class HipKernels(Kernels):
 
     # out[t, :] = table[tokens[t], :] * scale as float32
     # (add: out[t, :] += the same, for a stream that is shown its tokens' embeddings again)
-    def embed_rows(self, out: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor, scale: float = 1.0, add: bool = False) -> None:
+    # (waves = (positions, rates): feature 2i also gets the sine and 2i + 1 the cosine of positions[t] * rates[i], 32-bit)
+    def embed_rows(self, out: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor, scale: float = 1.0, add: bool = False, waves=None) -> None:
         assert out.dtype == torch.float32 and tokens.dtype == torch.int32 and table.is_contiguous() and out.is_contiguous()
         assert out.shape[0] == tokens.shape[0] and out.shape[1] == table.shape[1]
+        if waves is not None:
+            positions, rates = waves
+            assert not add and positions.dtype == torch.int32 and positions.shape[0] == out.shape[0]
+            assert rates.dtype == torch.float32 and rates.is_contiguous() and rates.numel() == (out.shape[1] + 1) // 2
+            return self._run("embed with positions", out.numel() * (4 + table.element_size()), 40 * out.numel(), None, self.lib.llmrs_embed_rows_waves,
+                             self._stream(), _code(table.dtype), _p(out), _p(table), _p(tokens), tokens.shape[0], table.shape[1], table.shape[0],
+                             float(scale), _p(positions), _p(rates))
         self._run("embed add" if add else "embed", out.numel() * ((8 if add else 4) + table.element_size()), out.numel() if add else 0, None,
                   self.lib.llmrs_embed_rows_add if add else self.lib.llmrs_embed_rows, self._stream(), _code(table.dtype), _p(out), _p(table), _p(tokens),
                   tokens.shape[0], table.shape[1], table.shape[0], float(scale))
@@ -347,6 +368,18 @@ class HipKernels(Kernels):
         self._run(f"rmsnorm {n}x{x.shape[1]}", n * x.shape[1] * (4 + out.element_size()) + x.shape[1] * 4, 5 * n * x.shape[1], None,
                   self.lib.llmrs_rmsnorm, self._stream(), _code(out.dtype), _p(out), _p(x), _p(weight), _p(rows),
                   n, x.shape[1], eps)
+
+    def post_norm(self, h: torch.Tensor, y: torch.Tensor, weight: Optional[torch.Tensor], x: Optional[torch.Tensor], eps: float = 0.0) -> None:
+        """h += rmsnorm(y) * weight (weight None: h stays), then x = h in x's type (x None: not wanted) and y = 0: the
+        norm of a sublayer's result y on its way into the stream h, and what the next sublayer needs.  h, y float32 [T, D]."""
+        T, D = h.shape
+        assert h.dtype == y.dtype == torch.float32 and h.is_contiguous() and y.is_contiguous() and y.shape == h.shape and h.data_ptr() != y.data_ptr()
+        assert weight is None or (weight.dtype == torch.float32 and weight.numel() == D and weight.is_contiguous() and eps > 0)
+        assert x is None or (x.shape == h.shape and x.is_contiguous() and x.data_ptr() != h.data_ptr())
+        xb = 0 if x is None else x.element_size()
+        self._run(f"post_norm {T}x{D}" if weight is not None else f"stream_rows {T}x{D}", T * D * ((16 if weight is not None else 8) + xb),
+                  6 * T * D, None, self.lib.llmrs_post_norm_rows, self._stream(), _code(torch.float32 if x is None else x.dtype), _p(h), _p(y),
+                  _p(weight), _p(x), T, D, float(eps))
 
     def dyt(self, out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, alpha: torch.Tensor,
             rows: Optional[torch.Tensor] = None, second=None) -> None:
@@ -528,8 +561,13 @@ class HipKernels(Kernels):
 
     def attention(self, q, out, k_cache, v_cache, block_table, token_entry, positions, q_starts, seq_lens,
                   n_heads, n_kv_heads, head_dim, page_size, num_pages, window, scale, scratch=None, max_seq_len=0, n_single=-1,
-                  single_keys=0, value_dim=0, distance=None, softcap=0.0, keep_first=0, sink=None, gate=None, gate_per=1) -> None:
-        """gate: float32 [T, n_heads * value_dim / gate_per] or None: every gate_per consecutive output features of a token
+                  single_keys=0, value_dim=0, distance=None, softcap=0.0, keep_first=0, sink=None, gate=None, gate_per=1,
+                  mask_chunk=0, difference=None) -> None:
+        """mask_chunk: > 0 (window 0): positions lie in chunks of so many, and a query sees its own chunk's keys only.
+        difference = (lambda, eps, scale): differential attention: a head's head_dim features of q and of a key are two
+        halves, each an attention of its own over the same values; with their results a1 and a2 the head's is
+        o = a1 - lambda a2, o / sqrt(mean(o^2) + eps) * scale.
+        gate: float32 [T, n_heads * value_dim / gate_per] or None: every gate_per consecutive output features of a token
         are multiplied by the sigmoid of their number (32-bit, before the one rounding).
         sink: float32 [n_heads] or None: the softmax's denominator of head h also holds exp(sink[h]), once for every
         query (a key without a value; not scaled).  single_keys: how many keys the single-token entries see together (windows counted), 0 if unknown.
@@ -541,10 +579,11 @@ class HipKernels(Kernels):
         assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous()
         v_dim = int(value_dim) or head_dim
         assert k_cache.numel() == num_pages * n_kv_heads * page_size * head_dim and v_cache.numel() == num_pages * n_kv_heads * page_size * v_dim
-        if v_dim != head_dim or distance is not None or softcap > 0 or (keep_first > 0 and window > 0) or sink is not None or gate is not None:
+        if v_dim != head_dim or distance is not None or softcap > 0 or (keep_first > 0 and window > 0) or sink is not None or gate is not None \
+                or mask_chunk > 0 or difference is not None:
             return self._attention_ext(q, out, k_cache, v_cache, block_table, token_entry, positions, q_starts, seq_lens, n_heads,
                                        n_kv_heads, head_dim, page_size, num_pages, window, scale, scratch, max_seq_len, n_single,
-                                       single_keys, v_dim, distance, softcap, keep_first, sink, gate, gate_per)
+                                       single_keys, v_dim, distance, softcap, keep_first, sink, gate, gate_per, mask_chunk, difference)
         T = q.shape[0]
         assert token_entry.shape[0] == T and positions.shape[0] == T and out.shape[0] == T
         moved = flops = 0
@@ -563,8 +602,11 @@ class HipKernels(Kernels):
 
     def _attention_ext(self, q, out, k_cache, v_cache, block_table, token_entry, positions, q_starts, seq_lens, n_heads,
                        n_kv_heads, head_dim, page_size, num_pages, window, scale, scratch, max_seq_len, n_single, single_keys,
-                       v_dim, distance, softcap=0.0, keep_first=0, sink=None, gate=None, gate_per=1) -> None:
+                       v_dim, distance, softcap=0.0, keep_first=0, sink=None, gate=None, gate_per=1, mask_chunk=0, difference=None) -> None:
         T = q.shape[0]
+        maps = 1 if difference is None else 2
+        lam, diff_eps, diff_scale = (0.0, 0.0, 0.0) if difference is None else difference
+        assert head_dim % maps == 0 and (mask_chunk == 0 or window == 0)
         assert gate is None or (gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape[0] == T and gate_per >= 1
                                 and (n_heads * v_dim) % gate_per == 0 and gate.shape[1] == n_heads * v_dim // gate_per)
         assert sink is None or (sink.dtype == torch.float32 and sink.numel() == n_heads and sink.is_contiguous())
@@ -576,9 +618,14 @@ class HipKernels(Kernels):
         moved = flops = 0
         if self.times is not None:
             keys = int(seq_lens.sum().item())
-            seen = int((positions + 1).sum().item()) if window <= 0 else int((positions + 1).clamp(max=window + keep_first).sum().item())
+            if mask_chunk > 0:              # (the keys of the chunks that the step's tokens lie in)
+                seen = int((positions % mask_chunk + 1).sum().item())
+                starts = (positions[q_starts[:-1].long()] // mask_chunk) * mask_chunk
+                keys = int((seq_lens - starts).sum().item())
+            else:
+                seen = int((positions + 1).sum().item()) if window <= 0 else int((positions + 1).clamp(max=window + keep_first).sum().item())
             moved = (keys * n_kv_heads * (head_dim + v_dim) + T * n_heads * (head_dim + v_dim)) * q.element_size()
-            flops = 2 * seen * n_heads * (head_dim + v_dim)
+            flops = 2 * seen * n_heads * (head_dim + maps * v_dim)
         self._run(f"attention {T} tokens" + (" (decode)" if n_single == block_table.shape[0] else ""), moved, flops, q.dtype,
                   self.lib.llmrs_attention_ext,
                   self._stream(), _code(q.dtype), _p(q), q.stride(0), _p(out), out.stride(0), _p(k_cache), _p(v_cache),
@@ -586,7 +633,7 @@ class HipKernels(Kernels):
                   block_table.shape[0], T, n_heads, n_kv_heads, head_dim, page_size, num_pages, window, scale,
                   _p(scratch), 0 if scratch is None else scratch.numel() * scratch.element_size(), int(max_seq_len),
                   int(n_single), int(single_keys), int(self.allow_mfma), v_dim, _p(r1), _p(r2), float(softcap), int(keep_first), _p(sink),
-                  _p(gate), 0 if gate is None else gate.stride(0), int(gate_per))
+                  _p(gate), 0 if gate is None else gate.stride(0), int(gate_per), int(mask_chunk), maps, float(lam), float(diff_eps), float(diff_scale))
 
     # out[i, :] = weight * groupnorm(sum_s w_in[s] * x[s][rows[i] or i, :]); x: [T, D] or [S, T, D] float32
     def group_rmsnorm(self, out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, eps: float, groups: int,
@@ -633,14 +680,17 @@ class HipKernels(Kernels):
     def qkv_finish(self, sums: torch.Tensor, bias: Optional[torch.Tensor], q: torch.Tensor, slot_map, k_cache, v_cache,
                    n_heads: int, n_kv_heads: int, head_dim: int, v_dim: int, page_size: int, num_pages: int, write_kv: bool,
                    eps: float, positions: Optional[torch.Tensor] = None, inv_freq: Optional[torch.Tensor] = None, rotary_dim: int = 0,
-                   q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None, gain: float = 1.0, conv=None) -> None:
+                   q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None, gain: float = 1.0, conv=None,
+                   maps: int = 1) -> None:
         """sums [T, q | k | v] float32 -> q [T, heads * head_dim] (activation type) and the cache's pages: biases
         added, q and k divided by their root mean square over the head (eps > 0) and multiplied by q_weight / k_weight
         [head_dim] (if given), then (rotary_dim > 0) their features (2i, 2i + 1) turned by positions[t] * inv_freq[i],
         cosine and sine times `gain`; one rounding on the way out.
         conv = (taps [columns, K] float32, state [slots, >= (K - 1) * columns] float32 or None when K == 1, q_starts, slots,
         token_entry): every column first passes a causal convolution over its K taps, the last tap the token's own; rows
-        before an entry's first token come from the request's state (which `conv_state_update` brings up to date afterwards)."""
+        before an entry's first token come from the request's state (which `conv_state_update` brings up to date afterwards).
+        maps = 2: every head of q and k is two of head_dim features, each normed and turned by itself; a key's two halves
+        lie side by side in a cache row of 2 head_dim."""
         taps = state = q_starts = slots = token_entry = None
         n_taps = n_entries = 0
         if conv is not None:
@@ -656,11 +706,11 @@ class HipKernels(Kernels):
             assert positions.dtype == torch.int32 and positions.shape[0] == sums.shape[0] and inv_freq.dtype == torch.float32
             assert inv_freq.shape[0] == rotary_dim // 2 and inv_freq.is_contiguous() and rotary_dim % 2 == 0 and rotary_dim <= head_dim
         assert sums.dtype == torch.float32 and sums.stride(1) == 1 and q.stride(1) == 1 and q.shape[0] == sums.shape[0]
-        width = (n_heads + n_kv_heads) * head_dim + n_kv_heads * v_dim
-        assert sums.shape[1] == width and (bias is None or (bias.dtype == torch.float32 and bias.numel() == width and bias.is_contiguous()))
+        width = (n_heads + n_kv_heads) * maps * head_dim + n_kv_heads * v_dim
+        assert sums.shape[1] == width and q.shape[1] >= n_heads * maps * head_dim and (bias is None or (bias.dtype == torch.float32 and bias.numel() == width and bias.is_contiguous()))
         if write_kv:
             assert k_cache.dtype == v_cache.dtype == q.dtype and k_cache.is_contiguous() and v_cache.is_contiguous()
-            assert k_cache.numel() == num_pages * n_kv_heads * page_size * head_dim and v_cache.numel() == num_pages * n_kv_heads * page_size * v_dim
+            assert k_cache.numel() == num_pages * n_kv_heads * page_size * maps * head_dim and v_cache.numel() == num_pages * n_kv_heads * page_size * v_dim
             assert slot_map.dtype == torch.int32 and slot_map.shape[0] == sums.shape[0]
         T = sums.shape[0]
         self._run("qkv_finish", T * width * (4 + q.element_size()), 4 * T * width, None, self.lib.llmrs_qkv_finish,
@@ -668,7 +718,7 @@ class HipKernels(Kernels):
                   _p(k_cache), _p(v_cache), T, n_heads, n_kv_heads, head_dim, v_dim, page_size, num_pages, int(write_kv), float(eps),
                   _p(positions) if rotary_dim else None, _p(inv_freq) if rotary_dim else None, int(rotary_dim),
                   _p(q_weight), _p(k_weight), float(gain), _p(taps), int(n_taps), _p(state) if n_taps > 1 else None,
-                  state.stride(0) if n_taps > 1 else 0, _p(q_starts), _p(slots), _p(token_entry), int(n_entries))
+                  state.stride(0) if n_taps > 1 else 0, _p(q_starts), _p(slots), _p(token_entry), int(n_entries), int(maps))
 
     def add_bias_rows(self, rows: torch.Tensor, bias: torch.Tensor) -> None:
         """rows[t, :] += bias; both float32."""
@@ -792,19 +842,20 @@ class HipKernels(Kernels):
                   self.lib.llmrs_rmsnorm_sum, self._stream(), _p(out), *flat, T, D, float(coef), float(eps))
 
     def route_topk(self, logits: torch.Tensor, weights: torch.Tensor, top: int, renormalize: bool = False, score: str = "softmax",
-                   correction: Optional[torch.Tensor] = None, scale: float = 1.0) -> None:
+                   correction: Optional[torch.Tensor] = None, scale: float = 1.0, groups: int = 1, keep_groups: int = 1) -> None:
         """weights[t, e] = softmax(logits[t])[e] for the `top` experts with the largest scores (of equal ones the lower
         index), 0 for the others; with `renormalize` divided by the chosen scores' sum.  Both float32 [T, experts].
         score = "sigmoid": an expert's score is sigmoid(logit); the choice goes by score + correction [experts] (None:
         by the score), the weight is the score without it (with `renormalize` divided by the chosen scores' sum + 1e-20),
-        times scale."""
+        times scale.  groups > 1: the experts form so many equal groups of neighbours, and only those of the keep_groups
+        best groups can be chosen (a group is as good as its best expert)."""
         assert logits.dtype == weights.dtype == torch.float32 and logits.stride(1) == weights.stride(1) == 1 and logits.shape == weights.shape
         T, E = logits.shape
         kind = {"softmax": 0, "sigmoid": 1}[score]
         assert correction is None or (kind == 1 and correction.dtype == torch.float32 and correction.numel() == E and correction.is_contiguous())
         assert kind == 1 or scale == 1.0
         self._run(f"route_topk {T}x{E}", T * E * 8, 8 * T * E, None, self.lib.llmrs_route_topk, self._stream(), _p(logits),
-                  logits.stride(0), _p(weights), weights.stride(0), T, E, int(top), int(bool(renormalize)), kind, _p(correction), float(scale))
+                  logits.stride(0), _p(weights), weights.stride(0), T, E, int(top), int(bool(renormalize)), kind, _p(correction), float(scale), int(groups), int(keep_groups))
 
     def route_counts(self, weights: torch.Tensor, counts: torch.Tensor) -> None:
         """counts[e] = how many tokens chose expert e (weights[t, e] > 0); weights float32 [T, E], counts int32 [E]."""
@@ -837,12 +888,13 @@ class HipKernels(Kernels):
                    limit: float = 0.0, alpha: float = 1.0) -> None:
         """out[t, c] = act * (weights[t, c // ff] if weights is given); up, weights float32.  "relu2": act =
         relu(up[t, c])^2.  "clamped_glu": up holds (gate, up) side by side, [T, 2 N]; with g = min(up[t, 2c], limit) and
-        u = clamp(up[t, 2c + 1], -limit, limit), act = g sigmoid(alpha g) (u + 1)."""
+        u = clamp(up[t, 2c + 1], -limit, limit), act = g sigmoid(alpha g) (u + 1).  "swiglu": the same layout, act =
+        silu(up[t, 2c]) up[t, 2c + 1]."""
         T, N = out.shape
-        kind = {"relu2": 0, "clamped_glu": 1}[activation]
-        assert up.dtype == torch.float32 and up.stride(1) == 1 and up.shape == (T, N * (2 if kind == 1 else 1)) and out.stride(1) == 1 and N % ff == 0
+        kind = {"relu2": 0, "clamped_glu": 1, "swiglu": 2}[activation]
+        assert up.dtype == torch.float32 and up.stride(1) == 1 and up.shape == (T, N * (2 if kind > 0 else 1)) and out.stride(1) == 1 and N % ff == 0
         assert weights is None or (weights.dtype == torch.float32 and weights.stride(1) == 1 and tuple(weights.shape) == (T, N // ff))
-        self._run(f"act_weight {T}x{N}", T * N * (4 * (kind + 1) + out.element_size()), (3 + 8 * kind) * T * N, None,
+        self._run(f"act_weight {T}x{N}", T * N * (4 * (2 if kind > 0 else 1) + out.element_size()), (3 + 8 * (kind > 0)) * T * N, None,
                   self.lib.llmrs_act_weight, self._stream(), _code(out.dtype), _p(up), up.stride(0), _p(weights),
                   0 if weights is None else weights.stride(0), int(ff), T, N, kind, _p(out), out.stride(0), float(limit), float(alpha))
 

@@ -26,7 +26,14 @@ rows ride in the q/k/v product), `qk_norm_scope` = "projection" (the q/k norm ru
 at once, with a weight of that width, instead of head by head), `value_mix` = "first" | "later" (the values of a
 "later" layer become (1 - lambda) v + lambda v_first before they are cached, v_first the values that the "first" such
 layer made of the same token in the same step and lambda the layer's one number, tensor leaf `vmix`; the "first" layer
-holds the tensor too and does not use it), `names` (the leaves of the tensors' names).  With any of them the q/k/v product leaves
+holds the tensor too and does not use it), `mask_chunk` (positions lie in chunks of so many, counted from the request's
+position 0, and a query sees its own chunk's keys only; no window then), `cache_window` (how many of a request's latest
+positions the cache has to hold, where that is more than the mixer's own mask needs: other mixers read this one's cache
+through masks of their own), `difference` = {base, eps} (differential attention: every head of q and of k is two maps of
+head_dim features, k's two side by side in a cache row of 2 head_dim; each map is an attention of its own over the same
+values, and with their results a1 and a2 the head's is o = a1 - lambda a2, divided by its root mean square, times 1 - base;
+lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + base, one number a layer, from four tensors of head_dim numbers), `names` (the
+leaves of the tensors' names).  With any of them the q/k/v product leaves
 32-bit sums, and one kernel convolves, adds the biases, norms q and k, rotates them (a rotation that the kernels fuse,
 angles in 32-bit) and writes k and v into their pages.
 
@@ -49,7 +56,8 @@ from .base import Mixer, TensorSpec, build_position, place, register_mixer
 
 class KeyedBySplitChunk:
     """For mixers that call `kernels().attention`: what their recordings are keyed by.  The mixer sets
-    `recording_signature = ("attention", kv_heads, head_dim, window)`, the shape of the cache its queries walk."""
+    `recording_signature = ("attention", kv_heads, head_dim, window, mask_chunk)`, the shape of the cache its queries walk
+    and how much of it they see (the chunk may be left out: 0)."""
 
     # The kernel library shares the decoding requests' keys out over waves in chunks whose length it chooses by
     # how many keys the step sees (`single_keys`).  A recorded step holds the chunk it was recorded with, so the
@@ -62,7 +70,7 @@ class KeyedBySplitChunk:
         k = kernels()
         if not ctx.n_single:
             return 0
-        keys = ctx.single_keys(self.recording_signature[3])
+        keys = ctx.single_keys(*self.recording_signature[3:])
         want = k.attention_split_chunk(ctx.n_single, self.recording_signature[1], self.recording_signature[2], ctx.max_seq_len, keys)
         held = ctx.part_state.setdefault(self.recording_signature, {})
         at = (ctx.n_single, ctx.max_seq_len)
@@ -80,7 +88,7 @@ class KeyedBySplitChunk:
         now = ctx.part_state.get(self.recording_signature, {}).get((ctx.n_single, ctx.max_seq_len))
         if now is not None and now[3] == ctx.serial:      # this step was keyed by a chunk: the figure that gives it
             return now[1]
-        return ctx.single_keys(self.recording_signature[3])
+        return ctx.single_keys(*self.recording_signature[3:])
 
 
 class Attention(KeyedBySplitChunk, Mixer):
@@ -94,7 +102,19 @@ class Attention(KeyedBySplitChunk, Mixer):
         self.kv_heads = int(p["num_kv_heads"])
         self.head_dim = int(p["head_dim"])
         self.window = int(p.get("window") or 0)
-        self.recording_signature = ("attention", self.kv_heads, self.head_dim, self.window)
+        self.mask_chunk = int(p.get("mask_chunk") or 0)
+        if self.mask_chunk < 0 or (self.mask_chunk > 0 and self.window > 0):
+            raise ValueError("a mask in chunks has a positive size and goes without a window")
+        self.cache_window = max(int(p.get("cache_window") or 0), self.window, self.mask_chunk) if self.window or self.mask_chunk else 0
+        difference = p.get("difference")
+        self.maps = 1 if difference is None else 2
+        self.key_dim = self.maps * self.head_dim             # a head's row of q, and a key's row in the cache
+        self.diff_base = self.diff_eps = 0.0
+        if difference is not None:
+            self.diff_base, self.diff_eps = float(difference["base"]), float(difference["eps"])
+            if not self.diff_eps > 0:
+                raise ValueError("the norm of the maps' difference needs a positive eps")
+        self.recording_signature = ("attention", self.kv_heads, self.key_dim, self.window, self.mask_chunk)
         self.kv_proj = bool(p.get("kv_proj", True))
         scale = p.get("scale")
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.head_dim)
@@ -103,8 +123,8 @@ class Attention(KeyedBySplitChunk, Mixer):
             self.graph_safe = False      # its apply() is free to do anything
         if self.heads % self.kv_heads:
             raise ValueError(f"{self.heads} heads are no multiple of {self.kv_heads} kv heads")
-        self.q_size = self.heads * self.head_dim
-        self.kv_size = self.kv_heads * self.head_dim
+        self.q_size = self.heads * self.key_dim
+        self.kv_size = self.kv_heads * self.key_dim
         self.value_dim = int(p.get("value_dim") or self.head_dim)
         self.v_size = self.kv_heads * self.value_dim
         self.o_size = self.heads * self.value_dim
@@ -138,6 +158,9 @@ class Attention(KeyedBySplitChunk, Mixer):
         if (self.norm_whole or self.value_mix is not None) and (self.taps > 0 or self.has_bias):
             raise ValueError("a q/k norm over the whole projection and a mix of values work on the projection's sums as they are: "
                              "with neither convolutions nor biases")
+        if self.maps > 1 and (self.distance is not None or self.softcap > 0 or self.keep_first > 0 or self.norm_whole or self.value_mix is not None):
+            raise ValueError("differential attention with a distance penalty, a soft cap, kept first keys, a q/k norm over the whole "
+                             "projection or mixed values is not built")
         if self.taps > 0 and (not self.kv_proj or self.has_bias):
             raise ValueError("convolutions on q, k and v go with neither biases nor a cache that another mixer wrote")
         self.gate_size = {None: 0, "feature": self.o_size, "head": self.heads}[self.gate]
@@ -145,19 +168,22 @@ class Attention(KeyedBySplitChunk, Mixer):
         # q and k are prepared by a kernel of their own between the product and attention
         self.prepared = (self.has_bias or self.qk_norm_eps > 0 or self.distance is not None or self.value_dim != self.head_dim
                          or self.softcap > 0 or self.keep_first > 0 or self.taps > 1 or self.gate is not None or self.gain != 1.0
-                         or self.value_mix is not None)
+                         or self.value_mix is not None or self.mask_chunk > 0 or self.maps > 1)
         if self.prepared and self.position is not None and self.position.rotary() is None:
             raise ValueError("a position encoding that is no rotation together with biases, a q/k norm, a distance penalty, a soft cap, "
                              "kept first keys or values of another width is not built")
         leaves = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
                   "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias", "r1": "r1", "r2": "r2",
                   "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "q_conv": "q_conv.weight", "k_conv": "k_conv.weight",
-                  "v_conv": "v_conv.weight", "gate": "gate_proj.weight", "value_mix": "vmix", **(p.get("names") or {})}
+                  "v_conv": "v_conv.weight", "gate": "gate_proj.weight", "value_mix": "vmix", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2",
+                  **(p.get("names") or {})}
         self.names = {key: self.name(leaf) for key, leaf in leaves.items()}
         self.w_qkv = None
         self.w_o = None
         self.bias = self.o_bias = self.r1 = self.r2 = None
         self.q_norm = self.k_norm = self.conv = self.mix = None
+        self.diff_vectors = None        # the four vectors that lambda is made of, as the file has them (on the host), and lambda
+        self.diff_lambda = 0.0
         # Set by a part that holds this mixer and adds the output projection's bias itself, in a pass over the output
         # that it makes anyway (it reads the bias from `o_bias`): `forward` then leaves the bias out.
         self.output_bias_left_to_holder = False
@@ -190,6 +216,8 @@ class Attention(KeyedBySplitChunk, Mixer):
             t[n["v_conv"]] = TensorSpec((self.v_size, self.taps), "normal:0.0:0.4")
         if self.gate is not None:
             t[n["gate"]] = TensorSpec((self.gate_size, self.hidden))
+        if self.maps > 1:
+            t.update({n[key]: TensorSpec((self.head_dim,), "normal:0.0:0.1") for key in ("lq1", "lk1", "lq2", "lk2")})
         return t
 
     def _pair_neighbours(self, w: torch.Tensor, heads: int, undo: bool = False) -> torch.Tensor:
@@ -207,38 +235,46 @@ class Attention(KeyedBySplitChunk, Mixer):
     def load(self, tensors, device):
         get = lambda n: place(tensors[self.names[n]], device, self.dtype)
         get32 = lambda n: place(tensors[self.names[n]], device, torch.float32)
-        parts = [self._pair_neighbours(get("q"), self.heads)]
+        hq, hk = self.heads * self.maps, self.kv_heads * self.maps
+        parts = [self._pair_neighbours(get("q"), hq)]
         if self.kv_proj:
-            parts += [self._pair_neighbours(get("k"), self.kv_heads), get("v")]
+            parts += [self._pair_neighbours(get("k"), hk), get("v")]
         self.qkv_width = sum(w.shape[0] for w in parts)
         if self.gate is not None:       # the gate's rows behind q | k | v: one product for all that reads the mixer's input
             parts.append(get("gate"))
         self.w_qkv = torch.cat(parts, dim=0).contiguous()
         self.w_o = get("o")
         if self.qk_norm_weight:         # (a head's features are listed in the order its rotation pairs them in)
-            hq, hk = (self.heads, self.kv_heads) if self.norm_whole else (1, 1)
-            self.q_norm = self._pair_neighbours(get32("q_norm").unsqueeze(1), hq).squeeze(1).contiguous()
-            self.k_norm = self._pair_neighbours(get32("k_norm").unsqueeze(1), hk).squeeze(1).contiguous() if self.kv_proj else None
+            nq, nk = (self.heads, self.kv_heads) if self.norm_whole else (1, 1)
+            self.q_norm = self._pair_neighbours(get32("q_norm").unsqueeze(1), nq).squeeze(1).contiguous()
+            self.k_norm = self._pair_neighbours(get32("k_norm").unsqueeze(1), nk).squeeze(1).contiguous() if self.kv_proj else None
         if self.value_mix is not None:
             self.mix = get32("value_mix").reshape(1)        # stays on the device: the kernel reads it there
         if self.taps > 0:               # the taps of q | k | v one under the other, as the product's columns are
-            self.conv = torch.cat([self._pair_neighbours(get32("q_conv"), self.heads), self._pair_neighbours(get32("k_conv"), self.kv_heads),
+            self.conv = torch.cat([self._pair_neighbours(get32("q_conv"), hq), self._pair_neighbours(get32("k_conv"), hk),
                                    get32("v_conv")], dim=0).contiguous()
         if self.has_bias:       # added to the 32-bit sums: kept in 32-bit, side by side as the product's columns are (and reordered as its rows are)
             pair = lambda b, heads: self._pair_neighbours(b.unsqueeze(1), heads).squeeze(1)
-            self.bias = torch.cat([pair(get32("q_bias"), self.heads)] +
-                                  ([pair(get32("k_bias"), self.kv_heads), get32("v_bias")] if self.kv_proj else [])).contiguous()
+            self.bias = torch.cat([pair(get32("q_bias"), hq)] +
+                                  ([pair(get32("k_bias"), hk), get32("v_bias")] if self.kv_proj else [])).contiguous()
         if self.has_o_bias:
             self.o_bias = get32("o_bias")
         if self.distance is not None:
             self.r1, self.r2 = get32("r1"), get32("r2")
+        if self.maps > 1:               # one number for the layer, made once
+            self.diff_vectors = {key: place(tensors[self.names[key]], "cpu", torch.float32) for key in ("lq1", "lk1", "lq2", "lk2")}
+            dot = lambda a, b: float((self.diff_vectors[a].double() * self.diff_vectors[b].double()).sum())
+            self.diff_lambda = math.exp(dot("lq1", "lk1")) - math.exp(dot("lq2", "lk2")) + self.diff_base
         if self.position is not None:
             self.position.to(device)
 
     def export(self):
         w = self.w_qkv.cpu()
         n = self.names
-        out = {n["q"]: self._pair_neighbours(w[:self.q_size], self.heads, undo=True).contiguous(), n["o"]: self.w_o.cpu()}
+        heads, kv_heads = self.heads * self.maps, self.kv_heads * self.maps
+        out = {n["q"]: self._pair_neighbours(w[:self.q_size], heads, undo=True).contiguous(), n["o"]: self.w_o.cpu()}
+        if self.maps > 1:
+            out.update({n[key]: v for key, v in self.diff_vectors.items()})
         if self.gate is not None:
             out[n["gate"]] = w[self.qkv_width:].contiguous()
         if self.qk_norm_weight:
@@ -250,19 +286,19 @@ class Attention(KeyedBySplitChunk, Mixer):
             out[n["value_mix"]] = self.mix.cpu().reshape(())
         if self.taps > 0:
             c = self.conv.cpu()
-            out[n["q_conv"]] = self._pair_neighbours(c[:self.q_size], self.heads, undo=True).contiguous()
-            out[n["k_conv"]] = self._pair_neighbours(c[self.q_size:self.q_size + self.kv_size], self.kv_heads, undo=True).contiguous()
+            out[n["q_conv"]] = self._pair_neighbours(c[:self.q_size], heads, undo=True).contiguous()
+            out[n["k_conv"]] = self._pair_neighbours(c[self.q_size:self.q_size + self.kv_size], kv_heads, undo=True).contiguous()
             out[n["v_conv"]] = c[self.q_size + self.kv_size:].contiguous()
         if self.kv_proj:
             k, v = w[self.q_size:self.q_size + self.kv_size], w[self.q_size + self.kv_size:self.qkv_width]
-            out[n["k"]] = self._pair_neighbours(k, self.kv_heads, undo=True).contiguous()
+            out[n["k"]] = self._pair_neighbours(k, kv_heads, undo=True).contiguous()
             out[n["v"]] = v.contiguous()
         if self.has_bias:
             b = self.bias.cpu()
             unpair = lambda x, heads: self._pair_neighbours(x.unsqueeze(1), heads, undo=True).squeeze(1).contiguous()
-            out[n["q_bias"]] = unpair(b[:self.q_size], self.heads)
+            out[n["q_bias"]] = unpair(b[:self.q_size], heads)
             if self.kv_proj:
-                out[n["k_bias"]] = unpair(b[self.q_size:self.q_size + self.kv_size], self.kv_heads)
+                out[n["k_bias"]] = unpair(b[self.q_size:self.q_size + self.kv_size], kv_heads)
                 out[n["v_bias"]] = b[self.q_size + self.kv_size:].contiguous()
         if self.has_o_bias:
             out[n["o_bias"]] = self.o_bias.cpu()
@@ -271,7 +307,8 @@ class Attention(KeyedBySplitChunk, Mixer):
         return out
 
     def cache_need(self):
-        pages = PagedKV(self.kv_heads, self.head_dim, self.window, self.value_dim if self.value_dim != self.head_dim else 0, self.keep_first)
+        # (a mask in chunks of n never looks back over more than n - 1 positions: for what has to be held it is a window of n)
+        pages = PagedKV(self.kv_heads, self.key_dim, self.cache_window, self.value_dim if self.value_dim != self.key_dim else 0, self.keep_first)
         if self.taps > 1:       # beside the pages, in the request's slot: the last conv - 1 rows of q | k | v as projected, 32-bit
             return (pages, FixedState(((self.taps - 1) * self.qkv_columns,), torch.float32))
         return pages
@@ -312,18 +349,20 @@ class Attention(KeyedBySplitChunk, Mixer):
         conv = (self.conv, conv_state, ctx.q_starts, ctx.slots, ctx.token_entry) if self.taps > 0 else None
         k.qkv_finish(sums[:, :C], self.bias, q, ctx.slot_maps[g], cache.k, cache.v, self.heads, n_kv, self.head_dim, self.value_dim,
                      cache.page_size, cache.num_pages, write, eps, ctx.positions, inv_freq, rotary_dim,
-                     q_weight=q_weight, k_weight=k_weight, gain=self.gain, conv=conv)
+                     q_weight=q_weight, k_weight=k_weight, gain=self.gain, conv=conv, **({} if self.maps == 1 else {"maps": self.maps}))
         if self.taps > 1:
             k.conv_state_update(sums[:, :C], conv_state, ctx.q_starts, ctx.slots, C, self.taps)
         o = ctx.workspace("attn.out", (T, self.o_size), self.dtype)
-        need = k.attention_scratch_floats(ctx.n_entries, self.heads, max(self.head_dim, self.value_dim), ctx.max_seq_len,
+        need = k.attention_scratch_floats(ctx.n_entries, self.heads * self.maps, max(self.key_dim, self.value_dim), ctx.max_seq_len,
                                           self.kv_heads, ctx.n_single) if ctx.n_single else 0
         scratch = ctx.workspace("attn.partial", (need,), torch.float32) if need else None
         k.attention(q, o, cache.k, cache.v, ctx.block_tables[g], ctx.token_entry, ctx.positions, ctx.q_starts, ctx.seq_lens,
-                    self.heads, self.kv_heads, self.head_dim, cache.page_size, cache.num_pages, self.window, self.scale,
+                    self.heads, self.kv_heads, self.key_dim, cache.page_size, cache.num_pages, self.window, self.scale,
                     scratch, ctx.max_seq_len, ctx.n_single, self._keys_for_the_split(ctx), value_dim=self.value_dim,
                     distance=None if self.distance is None else (self.r1, self.r2), softcap=self.softcap, keep_first=self.keep_first,
-                    gate=sums[:, self.qkv_width:] if self.gate is not None else None, gate_per=1 if self.gate == "feature" else self.value_dim)
+                    gate=sums[:, self.qkv_width:] if self.gate is not None else None, gate_per=1 if self.gate == "feature" else self.value_dim,
+                    **({} if self.mask_chunk == 0 else {"mask_chunk": self.mask_chunk}),
+                    **({} if self.maps == 1 else {"difference": (self.diff_lambda, self.diff_eps, 1.0 - self.diff_base)}))
         k.gemm(o, self.w_o, h, EPI_ACCUM_F32, ctx.gemm_workspace(o, self.w_o))
         if self.has_o_bias and not self.output_bias_left_to_holder:
             k.add_bias_rows(h, self.o_bias)

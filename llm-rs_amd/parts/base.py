@@ -109,6 +109,13 @@ class Norm(Part):
         """h += norm(y), both float32 [T, size]: the norm of a sublayer's output on its way into the stream."""
         raise NotImplementedError(f"{type(self).__name__} cannot norm a sublayer's output into the stream")
 
+    def add_normed_leaving_rows(self, ctx, y: torch.Tensor, h: torch.Tensor, x: Optional[torch.Tensor]) -> None:
+        """`add_normed`, then x = h in x's type (x None: not wanted) and y cleared: what the next sublayer reads, where it
+        reads the stream itself, and what it adds into."""
+        from ..kernels import kernels
+        self.add_normed(ctx, y, h)
+        kernels().post_norm(h, y, None, x)
+
     def deferred_weight(self) -> Optional[torch.Tensor]:
         """For a norm of the form x / rms(x) * weight: the float32 weight, which lets the product before it
         prepare its rows and the product after it finish them (`kernels.NextNorm`, `kernels.NormedRows`);

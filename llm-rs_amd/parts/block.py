@@ -4,11 +4,12 @@ halves, norms after the parts) is another subclass of `Block`, registered under
 its own name; the parts it needs beyond these four come under the names the
 layer's spec gives them in `extra`.  "sandwich": a norm before and after each half.
 "parallel": both halves read the stream as it was, each through a norm of its own or both through the one norm the
-layer has."""
+layer has.  "postnorm": a norm after each half only; the halves read the stream itself."""
 from __future__ import annotations
 
 import torch
 
+from ..kernels import StreamRows, kernels
 from .base import Block, register_block
 
 
@@ -102,3 +103,41 @@ class ParallelBlock(Block):
 
 
 register_block("parallel", ParallelBlock)
+
+
+class PostNormBlock(Block):
+    """A norm on each sublayer's result and none in front: h += post_mixer_norm(mixer(h)), then, where the layer has a
+    feed-forward, h += post_feed_forward_norm(feed_forward(h)).  A sublayer reads the stream's rows in the activation type
+    and adds its result into cleared 32-bit rows; the norm after it adds them into the stream in 32-bit and, in the same
+    launch, leaves the next sublayer (of this block or the next) its rows and its cleared room (`StreamRows`): only the
+    first block of a stack makes them with a launch of its own.  A 32-bit engine's sublayers read the stream in place."""
+    needs = ("mixer", "post_mixer_norm")
+    keeps_left_current = True       # what is left when `forward` returns was left by the norm that wrote the stream last
+
+    def __init__(self, named):
+        super().__init__(named)
+        self.post_mixer_norm = self.named["post_mixer_norm"]
+        self.post_feed_forward_norm = self.named.get("post_feed_forward_norm")
+        if self.feed_forward is not None and self.post_feed_forward_norm is None:
+            raise ValueError("block arrangement PostNormBlock needs a norm after its feed-forward (post_feed_forward_norm)")
+
+    def _half(self, ctx, h, post, run) -> None:
+        rows = ctx.left_for(h)
+        in_place = self.mixer.dtype == torch.float32
+        if not isinstance(rows, StreamRows) or rows.y.shape != h.shape:
+            rows = StreamRows(h if in_place else ctx.workspace("block.x", h.shape, self.mixer.dtype), ctx.workspace("block.y", h.shape, torch.float32))
+            kernels().post_norm(h, rows.room, None, None if in_place else rows.y)
+        ctx.note_left(h, None)          # (the sublayer's own products leave nothing for a norm: they do not write the stream)
+        ctx.upcoming_norm = None
+        run(rows.y, rows.room)
+        post.add_normed_leaving_rows(ctx, rows.room, h, None if in_place else rows.y)
+        ctx.note_left(h, rows)
+
+    def forward(self, ctx, h, cache):
+        self._half(ctx, h, self.post_mixer_norm, lambda x, y: self.mixer.forward(ctx, x, y, cache))
+        if self.feed_forward is not None:
+            self._half(ctx, h, self.post_feed_forward_norm, lambda x, y: self.feed_forward.forward(ctx, x, y))
+        ctx.upcoming_norm = None
+
+
+register_block("postnorm", PostNormBlock)

@@ -58,8 +58,9 @@ class SwiGLU(FeedForward):
 register_feed_forward("swiglu", SwiGLU)
 
 
-ACTIVATIONS = ("relu2", "clamped_glu")       # relu(x)^2; gated: g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)
-GATED = ("clamped_glu",)                     # activations of two projections, gate and up
+# relu(x)^2; gated: g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit); gated: silu(gate) up
+ACTIVATIONS = ("relu2", "clamped_glu", "swiglu")
+GATED = ("clamped_glu", "swiglu")            # activations of two projections, gate and up
 
 
 class ClampedGLU(FeedForward):
@@ -172,11 +173,12 @@ class RoutedFF(FeedForward):
     0.87 ms a layer in one product against 1.2 ms one by one; experts of 3584 x 4096 2.1 ms against 1.4 ms).
     Names: `router`, and `expert` with a place for the expert's number (e.g. "e{}").
 
-    Further parameters: `activation` = "clamped_glu" (with `limit`, `alpha`): the experts have a gate projection beside
+    Further parameters: `activation` = "clamped_glu" (with `limit`, `alpha`) or "swiglu": the experts have a gate projection beside
     the up projection (tensor leaf `gate`), a row of one after a row of the other in the matrix that lies under the other
     experts'; `score` = "sigmoid": each expert's score is the sigmoid of its logit by itself, the choice goes by score +
     `correction` (a tensor [experts], leaf `correction`, if `correction` is true) and the weights are the scores without
-    it (`renormalize`: divided by the chosen scores' sum), times `scale`; `shared` = {kind, prefix leaf, params}: a
+    it (`renormalize`: divided by the chosen scores' sum), times `scale`; `groups` = {count, keep}: the experts form `count`
+    equal groups of neighbours, and only those of the `keep` groups whose best expert is best can be chosen; `shared` = {kind, prefix leaf, params}: a
     feed-forward of any registered kind that every token passes beside its experts, added in."""
     graph_safe = True
     SORT_FROM_ROWS = 128
@@ -194,7 +196,7 @@ class RoutedFF(FeedForward):
         self.gated = self.activation in GATED
         self.up_rows = (2 if self.gated else 1) * self.inter       # rows of an expert's part of the up matrix
         self.limit, self.alpha = float(p.get("limit", 0.0)), float(p.get("alpha", 1.702))
-        if self.gated and not self.limit > 0:
+        if self.activation == "clamped_glu" and not self.limit > 0:
             raise ValueError(f"the activation's limit must be positive, got {self.limit}")
         self.score = p.get("score", "softmax")
         if self.score not in ("softmax", "sigmoid"):
@@ -205,6 +207,12 @@ class RoutedFF(FeedForward):
             raise ValueError("a correction of the choice and a scale of the weights go with sigmoid scores")
         if not 1 <= self.top <= self.experts:
             raise ValueError(f"top = {self.top} of {self.experts} experts")
+        groups = p.get("groups") or {"count": 1, "keep": 1}
+        self.groups, self.keep_groups = int(groups["count"]), int(groups["keep"])
+        if self.groups < 1 or self.experts % self.groups or not 1 <= self.keep_groups <= self.groups:
+            raise ValueError(f"{self.experts} experts do not fall into {self.groups} equal groups of which {self.keep_groups} are kept")
+        if self.top > self.experts // self.groups * self.keep_groups:
+            raise ValueError(f"top = {self.top} of the {self.experts // self.groups * self.keep_groups} experts of {self.keep_groups} groups")
         leaves = {"router": "router.weight", "expert": "experts.{}", "up": "up_proj.weight", "down": "down_proj.weight", "gate": "gate_proj.weight",
                   "correction": "correction", **(p.get("names") or {})}
         self.n_router = self.name(leaves["router"])
@@ -282,10 +290,11 @@ class RoutedFF(FeedForward):
         logits = ctx.workspace("moe.logits", (T, self.experts), torch.float32)
         k.gemm(x, self.w_router, logits, EPI_STORE_F32, ctx.gemm_workspace(x, self.w_router))
         weights = ctx.workspace("moe.weights", (T, self.experts), torch.float32)
+        groups = {} if self.groups == 1 else {"groups": self.groups, "keep_groups": self.keep_groups}
         if self.score == "sigmoid":
-            k.route_topk(logits, weights, self.top, self.renormalize, "sigmoid", self.correction, self.scale)
+            k.route_topk(logits, weights, self.top, self.renormalize, "sigmoid", self.correction, self.scale, **groups)
         else:
-            k.route_topk(logits, weights, self.top, self.renormalize)
+            k.route_topk(logits, weights, self.top, self.renormalize, **groups)
         if self.shared is not None:         # (reads x, adds into h; the experts' buffers are its own until it is done)
             self.shared.forward(ctx, x, h)
         if (self.w_down_each is not None and ctx.longest > 1 and T * self.top >= self.SORT_FROM_ROWS * self.experts

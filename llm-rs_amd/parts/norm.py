@@ -10,27 +10,35 @@ from .base import Norm, TensorSpec, place, register_norm
 
 
 class RMSNorm(Norm):
-    """`tensor`: the leaf of the weight's name ("weight"); "" when the prefix itself is the name."""
+    """`tensor`: the leaf of the weight's name ("weight"); "" when the prefix itself is the name.  `around_one`: the file
+    stores the weight's distance from one, y = x / rms(x) * (1 + w); the sum is made once, in 32-bit, when the weight is
+    taken."""
     graph_safe = True
 
     def __init__(self, spec, dtype):
         super().__init__(spec, dtype)
         self.size = int(spec.params["size"])
         self.eps = float(spec.params["eps"])
+        self.around_one = bool(spec.params.get("around_one", False))
         leaf = spec.params.get("tensor", "weight")
         self.weight_name = self.name(leaf) if leaf else self.prefix
         self.weight = None
+        self.stored = None          # (around_one: the weight as the file has it, which the sum does not give back exactly)
 
     def tensors(self):
-        return {self.weight_name: TensorSpec((self.size,), "norm")}
+        return {self.weight_name: TensorSpec((self.size,), "normal:0.0:0.1" if self.around_one else "norm")}
 
     def load(self, tensors, device):
         # The reference wants norm weights in 32-bit (ops.metal:972); whatever the
         # file stores, the kernel multiplies by a float32 weight.
-        self.weight = place(tensors[self.weight_name], device, torch.float32)
+        if self.around_one:
+            self.stored = place(tensors[self.weight_name], "cpu", torch.float32)
+            self.weight = (1.0 + self.stored).to(device)
+        else:
+            self.weight = place(tensors[self.weight_name], device, torch.float32)
 
     def export(self):
-        return {self.weight_name: self.weight.cpu()}
+        return {self.weight_name: self.stored if self.around_one else self.weight.cpu()}
 
     def forward(self, ctx, h, out, rows=None):
         kernels().rmsnorm(out, h, self.weight, self.eps, rows)
@@ -40,6 +48,9 @@ class RMSNorm(Norm):
 
     def add_normed(self, ctx, y, h):
         kernels().rmsnorm_sum(h, [(y, None, self.weight)], 1.0, self.eps)
+
+    def add_normed_leaving_rows(self, ctx, y, h, x):
+        kernels().post_norm(h, y, self.weight, x, self.eps)
 
     def deferred_weight(self):
         return self.weight

@@ -17,9 +17,20 @@ EPI_STORE, EPI_STORE_F32, EPI_ACCUM_F32, EPI_SWIGLU, EPI_GLU_CLAMP = 0, 1, 2, 3,
 class EmulatedKernels(Kernels):
     """(What `Kernels` answers by itself stays: no workspace, no scratch, nothing split.)"""
 
-    def embed_rows(self, out, table, tokens, scale=1.0, add=False):
+    def embed_rows(self, out, table, tokens, scale=1.0, add=False, waves=None):
         rows = table[tokens.long()].float() * scale
+        if waves is not None:
+            positions, rates = waves
+            angle = positions.float()[:, None] * rates[None, :]
+            rows += torch.stack([torch.sin(angle), torch.cos(angle)], dim=2).flatten(1)[:, :rows.shape[1]]
         out.add_(rows) if add else out.copy_(rows)
+
+    def post_norm(self, h, y, weight, x, eps=0.0):
+        if weight is not None:
+            h.add_(y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps) * weight)
+        y.zero_()
+        if x is not None:
+            x.copy_(h.to(x.dtype))
 
     def dyt(self, out, x, weight, bias, alpha, rows=None, second=None):
         src = x if rows is None else x[rows.long()]
@@ -194,7 +205,8 @@ class EmulatedKernels(Kernels):
 
     def attention(self, q, out, k_cache, v_cache, block_table, token_entry, positions, q_starts, seq_lens,
                   n_heads, n_kv_heads, head_dim, page_size, num_pages, window, scale, scratch=None, max_seq_len=0, n_single=-1,
-                  single_keys=0, value_dim=0, distance=None, softcap=0.0, keep_first=0, sink=None, gate=None, gate_per=1):
+                  single_keys=0, value_dim=0, distance=None, softcap=0.0, keep_first=0, sink=None, gate=None, gate_per=1,
+                  mask_chunk=0, difference=None):
         T = q.shape[0]
         v_dim = value_dim or head_dim
         kc = k_cache.view(num_pages, n_kv_heads, page_size, head_dim).float()
@@ -203,7 +215,7 @@ class EmulatedKernels(Kernels):
         for t in range(T):
             pos = int(positions[t])
             table = block_table[int(token_entry[t])]
-            lo = max(0, pos + 1 - window) if window > 0 else 0
+            lo = max(0, pos + 1 - window) if window > 0 else pos // mask_chunk * mask_chunk if mask_chunk > 0 else 0
             js = torch.cat([torch.arange(0, min(keep_first, lo)), torch.arange(lo, pos + 1)])
             pages, offs = table[js // page_size].long(), js % page_size
             assert int(pages.min()) >= 0, "a visible key's page was given back"
@@ -212,6 +224,16 @@ class EmulatedKernels(Kernels):
             qt = q[t, :n_heads * head_dim].view(n_heads, head_dim).float()
             for h in range(n_heads):
                 g = h // rep
+                if difference is not None:   # two maps over the same values, one taken off the other
+                    lam, diff_eps, diff_scale = difference
+                    half = head_dim // 2
+                    a = [torch.softmax((keys[:, g, m * half:(m + 1) * half] @ qt[h][m * half:(m + 1) * half]) * scale, dim=0) @ vals[:, g, :] for m in (0, 1)]
+                    o = a[0] - lam * a[1]
+                    o = o / torch.sqrt((o * o).mean() + diff_eps) * diff_scale
+                    if gate is not None:
+                        o = o * torch.sigmoid(gate[t, torch.arange(h * v_dim, (h + 1) * v_dim) // gate_per].float())
+                    out[t, h * v_dim:(h + 1) * v_dim] = o.to(out.dtype)
+                    continue
                 s = (keys[:, g, :] @ qt[h]) * scale
                 if softcap > 0:
                     s = softcap * torch.tanh(s / softcap)
@@ -237,8 +259,9 @@ class EmulatedKernels(Kernels):
             zero.zero_()
 
     def qkv_finish(self, sums, bias, q, slot_map, k_cache, v_cache, n_heads, n_kv_heads, head_dim, v_dim, page_size, num_pages,
-                   write_kv, eps, positions=None, inv_freq=None, rotary_dim=0, q_weight=None, k_weight=None, gain=1.0, conv=None):
+                   write_kv, eps, positions=None, inv_freq=None, rotary_dim=0, q_weight=None, k_weight=None, gain=1.0, conv=None, maps=1):
         T = sums.shape[0]
+        v_heads, n_heads, n_kv_heads = n_kv_heads, n_heads * maps, n_kv_heads * maps
         if conv is not None:
             taps, state, q_starts, slots, token_entry = conv
             K, C = taps.shape[1], sums.shape[1]
@@ -267,12 +290,12 @@ class EmulatedKernels(Kernels):
         q.copy_(qk[:, :n_heads].reshape(T, nq).to(q.dtype))
         if not write_kv:
             return
-        kc = k_cache.view(num_pages, n_kv_heads, page_size, head_dim)
-        vc = v_cache.view(num_pages, n_kv_heads, v_dim, page_size)
+        kc = k_cache.view(num_pages, v_heads, page_size, maps * head_dim)
+        vc = v_cache.view(num_pages, v_heads, v_dim, page_size)
         page, off = (slot_map // page_size).long(), (slot_map % page_size).long()
-        vals = x[:, nq + nk:].reshape(T, n_kv_heads, v_dim)
+        vals = x[:, nq + nk:].reshape(T, v_heads, v_dim)
         for t in range(T):
-            kc[page[t], :, off[t], :] = qk[t, n_heads:].to(kc.dtype)
+            kc[page[t], :, off[t], :] = qk[t, n_heads:].reshape(v_heads, maps * head_dim).to(kc.dtype)
             vc[page[t], :, :, off[t]] = vals[t].to(vc.dtype)
 
     def add_bias_rows(self, rows, bias):
@@ -342,10 +365,14 @@ class EmulatedKernels(Kernels):
             v = x if bias is None else x + bias
             out.add_(coef * v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * weight)
 
-    def route_topk(self, logits, weights, top, renormalize=False, score="softmax", correction=None, scale=1.0):
+    def route_topk(self, logits, weights, top, renormalize=False, score="softmax", correction=None, scale=1.0, groups=1, keep_groups=1):
         scores = torch.softmax(logits, dim=-1) if score == "softmax" else torch.sigmoid(logits)
         choice = scores if correction is None else scores + correction
         weights.zero_()
+        if groups > 1:
+            by_group = choice.view(choice.shape[0], groups, -1)
+            kept = torch.zeros(choice.shape[0], groups, dtype=torch.bool).scatter_(1, by_group.max(dim=2).values.topk(keep_groups, dim=1).indices, True)
+            choice = by_group.masked_fill(~kept[:, :, None], float("-inf")).reshape(choice.shape)
         for t in range(logits.shape[0]):
             chosen = sorted(range(logits.shape[1]), key=lambda e: (-float(choice[t, e]), e))[:top]
             total = (sum(float(scores[t, e]) for e in chosen) + (1e-20 if score == "sigmoid" else 0.0)) if renormalize else 1.0
@@ -356,6 +383,8 @@ class EmulatedKernels(Kernels):
         if activation == "clamped_glu":
             g, u = torch.clamp(up[:, 0::2], max=limit), torch.clamp(up[:, 1::2], min=-limit, max=limit)
             y = g * torch.sigmoid(alpha * g) * (u + 1.0)
+        elif activation == "swiglu":
+            y = up[:, 0::2] * torch.sigmoid(up[:, 0::2]) * up[:, 1::2]
         else:
             y = torch.clamp(up, min=0.0) ** 2
         if weights is not None:
