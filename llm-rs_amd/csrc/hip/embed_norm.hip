@@ -22,11 +22,17 @@ __device__ __forceinline__ bool rows_by_eights(const T* table, const float* out,
 // out[t, :] = float(table[tokens[t], :]) * scale   (reference: embed_batch_*, shaders/ops.metal:878-915,
 // which has no scale: 1 there and for every architecture that does not ask for one)
 // ADD: out[t, :] += the same, in 32-bit (a stream that is shown its tokens' embeddings again).
-// WAVES: a vector of the token's position is added, feature 2i the sine and 2i + 1 the cosine of positions[t] * rates[i],
-// angle, sine and cosine in 32-bit.
-__device__ __forceinline__ float position_wave(float pos, const float* __restrict__ rates, int d) {
-    float a = pos * rates[d >> 1];
-    return (d & 1) ? cosf(a) : sinf(a);
+// WAVES: a vector of the token's position is added, feature 2i the sine and 2i + 1 the cosine of positions[t] * rate i, in
+// 32-bit.  A rate is the sum of two 32-bit numbers, rates[i] and a small rates[n_rates + i]: what the product of position
+// and rate loses to rounding (thousands of turns leave few digits for the angle) is carried along and turns the result by
+// that little more.
+__device__ __forceinline__ void position_wave(float pos, float rate, float rate_rest, float& s, float& c) {
+    float a = pos * rate;
+    float rest = fmaf(pos, rate, -a) + pos * rate_rest;
+    float s0, c0;
+    sincosf(a, &s0, &c0);
+    s = fmaf(rest, c0, s0);
+    c = fmaf(-rest, s0, c0);
 }
 template <class T, bool ADD, bool WAVES>
 __global__ void embed_rows_kernel(float* __restrict__ out, const T* __restrict__ table,
@@ -34,6 +40,7 @@ __global__ void embed_rows_kernel(float* __restrict__ out, const T* __restrict__
                                   const int* __restrict__ positions, const float* __restrict__ rates) {
     int t = blockIdx.x;
     const float pos = WAVES ? (float)positions[t] : 0.0f;
+    const int n_rates = (D + 1) / 2;
     int row = tokens[t];
     row = row < 0 ? 0 : (row >= V ? V - 1 : row);  // the host has checked ids; never read outside the table
     const T* src = table + (size_t)row * D;
@@ -52,7 +59,7 @@ __global__ void embed_rows_kernel(float* __restrict__ out, const T* __restrict__
 #pragma unroll
                     for (int j = 0; j < 4; ++j) {
                         float s, c;
-                        sincosf(pos * rates[(d >> 1) + j], &s, &c);
+                        position_wave(pos, rates[(d >> 1) + j], rates[n_rates + (d >> 1) + j], s, c);
                         v[2 * j] += s;
                         v[2 * j + 1] += c;
                     }
@@ -64,7 +71,11 @@ __global__ void embed_rows_kernel(float* __restrict__ out, const T* __restrict__
     }
     for (int d = threadIdx.x; d < D; d += blockDim.x) {
         float v = (ADD ? dst[d] : 0.0f) + to_f32(src[d]) * scale;
-        if constexpr (WAVES) v += position_wave(pos, rates, d);
+        if constexpr (WAVES) {
+            float s, c;
+            position_wave(pos, rates[d >> 1], rates[n_rates + (d >> 1)], s, c);
+            v += (d & 1) ? c : s;
+        }
         dst[d] = v;
     }
 }
@@ -172,7 +183,7 @@ extern "C" int llmrs_embed_rows_add(hipStream_t stream, int dtype, float* out, c
     return embed_rows<true, false>(stream, dtype, out, table, tokens, n_tokens, D, V, scale);
 }
 
-// out[t, :] = float(table[tokens[t], :]) * scale + waves of positions[t] (see the kernel); rates: [(D + 1) / 2] 32-bit
+// out[t, :] = float(table[tokens[t], :]) * scale + waves of positions[t] (see the kernel); rates: [2][(D + 1) / 2] 32-bit
 extern "C" int llmrs_embed_rows_waves(hipStream_t stream, int dtype, float* out, const void* table, const int* tokens,
                                       int n_tokens, int D, int V, float scale, const int* positions, const float* rates) {
     LLMRS_REQUIRE(positions && rates, "embed_rows: the position vector needs positions and rates");

@@ -65,7 +65,8 @@ class Model:
         self.head = self.embedding if s.head_name is None else place(tensors[s.head_name], self.device, self.dtype)
         if s.position_wave_base > 0:
             i = torch.arange((s.hidden_size + 1) // 2, dtype=torch.float64)
-            self.wave_rates = torch.pow(torch.tensor(s.position_wave_base, dtype=torch.float64), -2.0 * i / s.hidden_size).float().to(self.device)
+            rates = torch.pow(torch.tensor(s.position_wave_base, dtype=torch.float64), -2.0 * i / s.hidden_size)
+            self.wave_rates = torch.stack([rates.float(), (rates - rates.float().double()).float()]).to(self.device)      # (as two 32-bit numbers each)
         for block in self.blocks:
             for part in block.parts():
                 part.load(tensors, self.device)

@@ -323,14 +323,15 @@ class HipKernels(Kernels):
 
     # out[t, :] = table[tokens[t], :] * scale as float32
     # (add: out[t, :] += the same, for a stream that is shown its tokens' embeddings again)
-    # (waves = (positions, rates): feature 2i also gets the sine and 2i + 1 the cosine of positions[t] * rates[i], 32-bit)
+    # (waves = (positions, rates [2, (width + 1) / 2]): feature 2i also gets the sine and 2i + 1 the cosine of
+    # positions[t] * (rates[0, i] + rates[1, i]), 32-bit)
     def embed_rows(self, out: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor, scale: float = 1.0, add: bool = False, waves=None) -> None:
         assert out.dtype == torch.float32 and tokens.dtype == torch.int32 and table.is_contiguous() and out.is_contiguous()
         assert out.shape[0] == tokens.shape[0] and out.shape[1] == table.shape[1]
         if waves is not None:
             positions, rates = waves
             assert not add and positions.dtype == torch.int32 and positions.shape[0] == out.shape[0]
-            assert rates.dtype == torch.float32 and rates.is_contiguous() and rates.numel() == (out.shape[1] + 1) // 2
+            assert rates.dtype == torch.float32 and rates.is_contiguous() and tuple(rates.shape) == (2, (out.shape[1] + 1) // 2)
             return self._run("embed with positions", out.numel() * (4 + table.element_size()), 40 * out.numel(), None, self.lib.llmrs_embed_rows_waves,
                              self._stream(), _code(table.dtype), _p(out), _p(table), _p(tokens), tokens.shape[0], table.shape[1], table.shape[0],
                              float(scale), _p(positions), _p(rates))

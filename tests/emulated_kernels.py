@@ -21,8 +21,8 @@ class EmulatedKernels(Kernels):
         rows = table[tokens.long()].float() * scale
         if waves is not None:
             positions, rates = waves
-            angle = positions.float()[:, None] * rates[None, :]
-            rows += torch.stack([torch.sin(angle), torch.cos(angle)], dim=2).flatten(1)[:, :rows.shape[1]]
+            angle = (positions.double()[:, None] * rates.double().sum(0)[None, :])
+            rows += torch.stack([torch.sin(angle), torch.cos(angle)], dim=2).flatten(1)[:, :rows.shape[1]].float()
         out.add_(rows) if add else out.copy_(rows)
 
     def post_norm(self, h, y, weight, x, eps=0.0):
