@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Decode and prefill throughput of the engine on one MI355X.
 
-    python bench.py --gpus 1 --steps K --warmup W [--workload decode8b|serve1b|mixed70b|sizes|sizes1b|prompts|long|widths|portions|tuvodra|lilatar|vivisun|gokosun]
+    python bench.py --gpus 1 --steps K --warmup W [--workload decode8b|serve1b|mixed70b|sizes|sizes1b|prompts|long|widths|portions|tuvodra|lilatar|vivisun|gokosun|tevovik]
 
 The default run (`decode8b`) is the Llama-3.1-8B shape with random bfloat16 weights: 8
 requests, each with 2,048 tokens of context in the cache, decode K steps through the
@@ -43,6 +43,9 @@ The other workloads print one line of the same form each:
             latent, a rotated key part and a sink, grouped-query attention with mixed values, a matrix memory with
             exponential gates, in threes; clamped gated feed-forwards, dense and as sigmoid-routed experts beside a
             shared one).
+  tevovik   the same for the Tevovik decoder (norms on the sublayers' results only; differential attention with half as many
+            heads of two maps each and values twice as wide, over chunks of positions, a third of the layers on the keys
+            and values of the layer before; gated experts chosen within groups).
 With LLM_PERF set in the environment every kernel call is timed by itself and a table
 by kernel goes to stderr (the reference's switch, src/backend/metal/mod.rs:235,321-400).
 """
@@ -73,7 +76,7 @@ LLAMA_8B = _llama(32, 4096, 32, 8, 128, 14336, 8.0, False)
 LLAMA_1B = _llama(16, 2048, 32, 8, 64, 8192, 32.0, True)
 LLAMA_70B = _llama(80, 8192, 64, 8, 128, 28672, 8.0, False)
 SHAPES = {"Llama-3.1-8B shape": LLAMA_8B, "Llama-3.2-1B shape": LLAMA_1B, "Llama-3.1-70B shape": LLAMA_70B}
-WORKLOADS = ("decode8b", "serve1b", "mixed70b", "sizes", "sizes1b", "prompts", "long", "widths", "portions", "tuvodra", "lilatar", "vivisun", "gokosun")
+WORKLOADS = ("decode8b", "serve1b", "mixed70b", "sizes", "sizes1b", "prompts", "long", "widths", "portions", "tuvodra", "lilatar", "vivisun", "gokosun", "tevovik")
 
 
 def flat_config(model: str, layers_run: int, global_batch: int, seq_len: int, page_size: int, **more) -> dict:
@@ -742,6 +745,39 @@ def run_gokosun(args) -> dict:
     return line
 
 
+def tevovik_shape(width, heads, kv_heads, dim, ff, chunk, repeats, experts, top, vocab=128256):
+    """Layers in threes, the second on the first's keys and values: differential attention with half as many heads as the
+    Llama shape, two maps of `dim` features and values of 2 dim each (the same q, k, v and output matrices), and experts in
+    four groups of which two are kept, the chosen ones together as wide as the dense feed-forward.
+    (The random table's rows are enlarged to the size of the position vector: else tokens at equal places choose equal experts.)"""
+    mix = lambda kv_from: {"heads": heads // 2, "kv_heads": kv_heads // 2, "dim": dim, "vdim": 2 * dim, "scale": dim ** -0.5, "diff": 0.4,
+                           "mask": {"size": chunk}, **({} if kv_from is None else {"kv_from": kv_from})}
+    groups = 4 if experts % 4 == 0 and top <= experts // 2 else 1
+    mlp = lambda: {"kind": "moe", "expert": {"ff": ff // top},
+                   "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": max(1, groups // 2)}}}
+    return {"architecture": "Tevovik", "vocab": vocab, "width": width, "embedding": {"scale": 50.0}, "norm": {"eps": 1e-6},
+            "layers": [{"type": "attention", "mixer": mix(3 * r if i == 1 else None), "mlp": mlp()} for r in range(repeats) for i in range(3)]}
+
+
+def run_tevovik(args) -> dict:
+    """Prompt and decode throughput of the Tevovik decoder at two widths, each beside a Llama decoder of the same
+    width, attention matrices, active feed-forward and number of layers (random weights both)."""
+    repeats = max(1, (args.layers or 6) // 3)
+    sizes = {"1B widths": (LLAMA_1B, 2048, 32, 8, 64, 8192), "8B widths": (LLAMA_8B, 4096, 32, 8, 128, 14336)}
+    pairs = {size: {"tevovik": tevovik_shape(width, heads, kv_heads, dim, ff, args.chunk, repeats, args.experts, args.top),
+                    "llama": dict(llama, num_hidden_layers=3 * repeats)}
+             for size, (llama, width, heads, kv_heads, dim, ff) in sizes.items()}
+    points = run_beside_llama(args, pairs, 3 * repeats)
+    first = next(iter(points.values()))
+    line = base_line("decode_tokens_per_s", first["decode_tokens_per_s"], args.steps, args.warmup, first["decode_ms_per_step"] * 1e-3, args.dtype,
+                     {"model": "Tevovik (differential attention over chunks of positions, every third layer on the cache of the one before; gated "
+                               "experts chosen within groups) beside Llama of equal widths",
+                      "global_batch": args.batch, "seq_len": args.context, "parallelism": "single GPU", "layers_run": 3 * repeats,
+                      "prefill_tokens": args.prefill_tokens, "chunk": args.chunk, "experts": args.experts, "top": args.top, "page_size": 16})
+    line["points"] = points
+    return line
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -760,11 +796,12 @@ def main() -> int:
     ap.add_argument("--new-tokens", type=int, default=256, help="serve1b: tokens generated for each request")
     ap.add_argument("--max-batch-tokens", type=int, default=2048, help="serve1b: tokens a scheduler step may run")
     ap.add_argument("--window", type=int, default=1024, help="tuvodra, lilatar: keys an attention layer sees")
-    ap.add_argument("--only-size", default="", help="tuvodra, lilatar, vivisun, gokosun: run one of the sizes only (1B or 8B)")
+    ap.add_argument("--chunk", type=int, default=4096, help="tevovik: positions of a chunk (the default: a prompt and its decoding lie in one)")
+    ap.add_argument("--only-size", default="", help="tuvodra, lilatar, vivisun, gokosun, tevovik: run one of the sizes only (1B or 8B)")
     ap.add_argument("--kv-rank", type=int, default=256, help="vivisun, gokosun: how many numbers a token of a latent layer leaves in the cache")
     ap.add_argument("--loop-times", type=int, default=1, help="vivisun: how often the layers after the first run in a row")
-    ap.add_argument("--experts", type=int, default=16, help="lilatar, gokosun: experts of a routed feed-forward")
-    ap.add_argument("--top", type=int, default=4, help="lilatar, gokosun: experts a token uses")
+    ap.add_argument("--experts", type=int, default=16, help="lilatar, gokosun, tevovik: experts of a routed feed-forward")
+    ap.add_argument("--top", type=int, default=4, help="lilatar, gokosun, tevovik: experts a token uses")
     ap.add_argument("--experts-by-rows-from", type=int, default=None,
                     help="lilatar: rows an expert gets on average from which a prompt step runs the experts one by one (default: the part's own rule)")
     args = ap.parse_args()
@@ -776,7 +813,7 @@ def main() -> int:
     args.warmup = args.warmup if args.warmup is not None else (2 if heavy else 8)
     line = {"decode8b": run_decode8b, "serve1b": run_serve1b, "mixed70b": run_mixed70b, "sizes": run_sizes, "sizes1b": run_sizes,
             "prompts": run_prompts, "long": run_long, "widths": run_widths, "portions": run_portions, "tuvodra": run_tuvodra, "lilatar": run_lilatar,
-            "vivisun": run_vivisun, "gokosun": run_gokosun}[args.workload](args)
+            "vivisun": run_vivisun, "gokosun": run_gokosun, "tevovik": run_tevovik}[args.workload](args)
     from llm_rs_amd.kernels import kernels
     if kernels().times is not None:         # LLM_PERF: what was still to be shown of the per-kernel table
         kernels().times.dump()

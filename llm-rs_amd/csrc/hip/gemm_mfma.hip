@@ -17,22 +17,7 @@
 // Replaces the reference's matvec_bf16_simd / gemm_bf16 (shaders/ops.metal:52-159,
 // :1090-1143); unlike gemm_bf16 (:1107) the accumulator is 32-bit.
 #include "cache_layout.h"
-#include "gemm.h"
-
-#include <type_traits>
-
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
-typedef float f32x4 __attribute__((ext_vector_type(4)));
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-
-template <int I, int N, class F>
-__device__ __forceinline__ void static_for(F&& f) {
-    if constexpr (I < N) {
-        f(std::integral_constant<int, I>{});
-        static_for<I + 1, N>(f);
-    }
-}
+#include "gemm_tile.h"
 
 __device__ __forceinline__ bf16x8 load8(const bf16* p) { return *(const bf16x8*)p; }
 __device__ __forceinline__ bf16x8 zero8() {
@@ -42,17 +27,6 @@ __device__ __forceinline__ bf16x8 zero8() {
     return z;
 }
 
-typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
-// The value the neighbouring lane (lane ^ 1) passes: a DPP move within each group of four lanes, no LDS.
-__device__ __forceinline__ float swap_neighbours(float x) {
-    int u = __float_as_int(x);
-    return __int_as_float(__builtin_amdgcn_update_dpp(u, u, 0xB1, 0xf, 0xf, true));     // quad_perm [1, 0, 3, 2]
-}
-// x / (1 + exp(-x)) with the device's exponential and reciprocal instructions (each within an ulp; the result is
-// rounded to bfloat16 right after).  For the epilogues that finish thousands of values per wave.
-__device__ __forceinline__ float silu_fast_f32(float x) {
-    return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -1.44269504088896341f));
-}
 // act(gate, up) of the gated epilogues with the same instructions; the clamped one's constants are read from their slot
 // once, before the loops that finish a tile (gated_act_of), not value by value
 struct GatedAct {
@@ -75,12 +49,6 @@ __device__ __forceinline__ float gated_act_fast(const GatedAct& a, float g, floa
     return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * a.alpha2)) * (u + 1.0f);
 }
 void llmrs_glu_clamp_store_mfma(hipStream_t stream, int slot, GluClamp p) { glu_clamp_store_kernel<<<1, 1, 0, stream>>>(slot, p); }
-
-// The tile loops' barrier: this wave's LDS reads and writes are done, then every wave of the block
-// has arrived.  Unlike __syncthreads() it does not wait for loads from memory that are still in
-// flight (the later tiles of a pipeline); the "memory" clobber keeps the compiler from moving
-// memory accesses across it.
-__device__ __forceinline__ void block_sync_lds() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 // ---------------------------------------------------------------------------
 // skinny: C^T[n, m] = sum_k W[n, k] X[m, k]
@@ -704,12 +672,6 @@ __device__ __forceinline__ void tile_epilogue(f32x16 (&acc)[BM / WGM / 32][BN / 
 // before this tile's products and waited for (s_waitcnt vmcnt) only as far as the
 // next tile needs.  No staging registers, no LDS store instructions.
 // ---------------------------------------------------------------------------
-template <int N_>
-__device__ __forceinline__ void wait_vmcnt() {
-    static_assert(N_ >= 0 && N_ < 64, "vmcnt is a 6-bit counter");
-    __builtin_amdgcn_s_waitcnt((N_ & 15) | (7 << 4) | (15 << 8) | ((N_ >> 4) << 14));
-}
-
 template <int BM, int BN, int WGM, int WGN, int STAGES>
 __global__ __launch_bounds__(64 * WGM * WGN) void gemm_dma_kernel(const bf16* __restrict__ A, int lda,
                                                        const bf16* __restrict__ W, void* __restrict__ out,

@@ -222,29 +222,45 @@ extern "C" int llmrs_act_weight(hipStream_t stream, int dtype, const float* up, 
 // ---- the experts' rows one after the other --------------------------------------------------------------------------
 // For steps of many tokens the chosen (token, expert) pairs are laid out expert by expert, each expert's rows in the
 // order of their tokens, so that an expert's tokens are a dense product of their own.  counts[e]: how many tokens chose
-// expert e (a wave an expert).  With the counts known: row_token[row], row_weight[row] for every row, and
-// row_of[t, e] = the row of token t with expert e, or -1 (a wave an expert; an expert's first row is the sum of the
-// counts before it).
-__global__ __launch_bounds__(64) void route_counts_kernel(const float* __restrict__ weights, int ldw, int T, int* __restrict__ counts) {
-    int e = blockIdx.x, lane = threadIdx.x, n = 0;
-    for (int t = lane; t < T; t += 64) n += weights[(size_t)t * ldw + e] > 0.0f;
+// expert e (a block an expert).  With the counts known: row_token[row], row_weight[row] for every row, and
+// row_of[t, e] = the row of token t with expert e, or -1 (a block an expert; an expert's first row is the sum of the
+// counts before it; each of its four waves takes a quarter of the tokens).
+#define ROUTE_ROW_WAVES 4
+__device__ __forceinline__ int chosen_in(const float* __restrict__ weights, int ldw, int e, int t_lo, int t_hi) {
+    int lane = threadIdx.x & 63, n = 0;
+#pragma unroll 4
+    for (int t = t_lo + lane; t < t_hi; t += 64) n += weights[(size_t)t * ldw + e] > 0.0f;
 #pragma unroll
     for (int d = 32; d > 0; d >>= 1) n += __shfl_xor(n, d, 64);
-    if (lane == 0) counts[e] = n;
+    return n;
+}
+__global__ __launch_bounds__(64 * ROUTE_ROW_WAVES) void route_counts_kernel(const float* __restrict__ weights, int ldw, int T, int* __restrict__ counts) {
+    __shared__ int part[ROUTE_ROW_WAVES];
+    int e = blockIdx.x, wave = threadIdx.x >> 6, per = (T + ROUTE_ROW_WAVES - 1) / ROUTE_ROW_WAVES;
+    int n = chosen_in(weights, ldw, e, wave * per, min(T, (wave + 1) * per));
+    if ((threadIdx.x & 63) == 0) part[wave] = n;
+    __syncthreads();
+    if (threadIdx.x == 0) counts[e] = part[0] + part[1] + part[2] + part[3];
 }
 
-__global__ __launch_bounds__(64) void route_rows_kernel(const float* __restrict__ weights, int ldw, int T, int E, const int* __restrict__ counts,
+__global__ __launch_bounds__(64 * ROUTE_ROW_WAVES) void route_rows_kernel(const float* __restrict__ weights, int ldw, int T, int E, const int* __restrict__ counts,
                                                          int* __restrict__ row_token, float* __restrict__ row_weight, int* __restrict__ row_of) {
-    int e = blockIdx.x, lane = threadIdx.x, first = 0;
+    __shared__ int part[ROUTE_ROW_WAVES];
+    int e = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, first = 0;
+    int per = (T + ROUTE_ROW_WAVES - 1) / ROUTE_ROW_WAVES, t_lo = wave * per, t_hi = min(T, t_lo + per);
+    int mine = chosen_in(weights, ldw, e, t_lo, t_hi);
+    if (lane == 0) part[wave] = mine;
     for (int i = lane; i < e; i += 64) first += counts[i];
 #pragma unroll
     for (int d = 32; d > 0; d >>= 1) first += __shfl_xor(first, d, 64);
-    for (int t0 = 0; t0 < T; t0 += 64) {
+    __syncthreads();
+    for (int w = 0; w < wave; ++w) first += part[w];
+    for (int t0 = t_lo; t0 < t_hi; t0 += 64) {
         int t = t0 + lane;
-        float w = t < T ? weights[(size_t)t * ldw + e] : 0.0f;
+        float w = t < t_hi ? weights[(size_t)t * ldw + e] : 0.0f;
         unsigned long long chosen = __ballot(w > 0.0f);
         int row = first + __popcll(chosen & ((1ull << lane) - 1ull));
-        if (t < T) row_of[(size_t)t * E + e] = w > 0.0f ? row : -1;
+        if (t < t_hi) row_of[(size_t)t * E + e] = w > 0.0f ? row : -1;
         if (w > 0.0f) { row_token[row] = t; row_weight[row] = w; }
         first += __popcll(chosen);
     }
@@ -252,7 +268,7 @@ __global__ __launch_bounds__(64) void route_rows_kernel(const float* __restrict_
 
 extern "C" int llmrs_route_counts(hipStream_t stream, const float* weights, int ldw, int n_tokens, int E, int* counts) {
     LLMRS_REQUIRE(weights && counts && E > 0 && ldw >= E && n_tokens >= 0 && E <= 65535, "route_counts: bad arguments");
-    route_counts_kernel<<<E, 64, 0, stream>>>(weights, ldw, n_tokens, counts);
+    route_counts_kernel<<<E, 64 * ROUTE_ROW_WAVES, 0, stream>>>(weights, ldw, n_tokens, counts);
     LLMRS_LAUNCH_CHECK("route_counts");
     return 0;
 }
@@ -260,7 +276,7 @@ extern "C" int llmrs_route_counts(hipStream_t stream, const float* weights, int 
 extern "C" int llmrs_route_rows(hipStream_t stream, const float* weights, int ldw, int n_tokens, int E, const int* counts, int* row_token,
                                 float* row_weight, int* row_of) {
     LLMRS_REQUIRE(weights && counts && row_token && row_weight && row_of && E > 0 && ldw >= E && n_tokens >= 0 && E <= 65535, "route_rows: bad arguments");
-    route_rows_kernel<<<E, 64, 0, stream>>>(weights, ldw, n_tokens, E, counts, row_token, row_weight, row_of);
+    route_rows_kernel<<<E, 64 * ROUTE_ROW_WAVES, 0, stream>>>(weights, ldw, n_tokens, E, counts, row_token, row_weight, row_of);
     LLMRS_LAUNCH_CHECK("route_rows");
     return 0;
 }
@@ -282,23 +298,47 @@ extern "C" int llmrs_gather_rows(hipStream_t stream, int dtype, void* out, int l
     return 0;
 }
 
-// h[t, :] += sum over the experts e that token t chose, in ascending e, of y[row_of[t, e], :]; 32-bit.
-__global__ void combine_rows_kernel(float* __restrict__ h, int ldh, const float* __restrict__ y, int ldy, const int* __restrict__ row_of, int E, int D) {
-    int t = blockIdx.x;
-    for (int d = threadIdx.x; d < D; d += blockDim.x) {
-        float acc = 0.0f;
-        for (int e = 0; e < E; ++e) {
-            int row = row_of[(size_t)t * E + e];
-            if (row >= 0) acc += y[(size_t)row * ldy + d];
+// h[t, :] += sum over the experts e that token t chose, in ascending e, of y[row_of[t, e], :]; 32-bit.  The token's rows are
+// listed first; VEC: rows of whole 16-byte pieces.
+template <bool VEC>
+__global__ __launch_bounds__(256) void combine_rows_kernel(float* __restrict__ h, int ldh, const float* __restrict__ y, int ldy,
+                                                           const int* __restrict__ row_of, int E, int D) {
+    __shared__ int list[ROUTE_MAX_EXPERTS];
+    int t = blockIdx.x, lane = threadIdx.x & 63, n = 0;
+    for (int base = 0; base < E; base += 64) {                  // (every wave makes the same list)
+        int row = base + lane < E ? row_of[(size_t)t * E + base + lane] : -1;
+        unsigned long long has = __ballot(row >= 0);
+        if (row >= 0 && threadIdx.x < 64) list[n + __popcll(has & ((1ull << lane) - 1ull))] = row;
+        n += __popcll(has);
+    }
+    __syncthreads();
+    if constexpr (VEC) {
+        for (int d = 4 * threadIdx.x; d < D; d += 1024) {
+            float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+            float4 old = *(const float4*)(h + (size_t)t * ldh + d);
+#pragma unroll 4
+            for (int i = 0; i < n; ++i) {
+                float4 v = *(const float4*)(y + (size_t)list[i] * ldy + d);
+                acc.x += v.x; acc.y += v.y; acc.z += v.z; acc.w += v.w;
+            }
+            *(float4*)(h + (size_t)t * ldh + d) = make_float4(old.x + acc.x, old.y + acc.y, old.z + acc.z, old.w + acc.w);
         }
-        h[(size_t)t * ldh + d] += acc;
+    } else {
+        for (int d = threadIdx.x; d < D; d += 256) {
+            float acc = 0.0f;
+            for (int i = 0; i < n; ++i) acc += y[(size_t)list[i] * ldy + d];
+            h[(size_t)t * ldh + d] += acc;
+        }
     }
 }
 
 extern "C" int llmrs_combine_rows(hipStream_t stream, float* h, int ldh, const float* y, int ldy, const int* row_of, int n_tokens, int E, int D) {
     LLMRS_REQUIRE(h && y && row_of && D > 0 && ldh >= D && ldy >= D && E > 0 && n_tokens >= 0, "combine_rows: bad arguments");
     if (n_tokens == 0) return 0;
-    combine_rows_kernel<<<n_tokens, 256, 0, stream>>>(h, ldh, y, ldy, row_of, E, D);
+    LLMRS_REQUIRE(E <= ROUTE_MAX_EXPERTS, "combine_rows: %d experts exceed %d", E, ROUTE_MAX_EXPERTS);
+    bool vec = D % 4 == 0 && ldh % 4 == 0 && ldy % 4 == 0 && ((uintptr_t)h & 15) == 0 && ((uintptr_t)y & 15) == 0;
+    if (vec) combine_rows_kernel<true><<<n_tokens, 256, 0, stream>>>(h, ldh, y, ldy, row_of, E, D);
+    else combine_rows_kernel<false><<<n_tokens, 256, 0, stream>>>(h, ldh, y, ldy, row_of, E, D);
     LLMRS_LAUNCH_CHECK("combine_rows");
     return 0;
 }

@@ -164,6 +164,11 @@ class Kernels:
         reads the stream next (`NextNorm`), or None: then a norm kernel runs."""
         return None
 
+    def grouped_experts_take(self, hidden: int, ff: int, dtype: torch.dtype) -> bool:
+        """Whether `expert_up` and `expert_down` (every expert's product over its own rows in one launch) and `expert_few_up` and
+        `expert_few_down` (up to 64 tokens; experts that none of them chose are not read) run experts of these sizes."""
+        return False
+
     def attention_scratch_floats(self, n_entries: int, n_heads: int, head_dim: int, max_seq_len: int,
                                  n_kv_heads: Optional[int] = None, n_single: int = 0) -> int:
         """Room (floats) for the partial results of single-token entries whose keys are shared out over waves."""
@@ -230,6 +235,11 @@ class HipKernels(Kernels):
             "llmrs_route_rows": [V, V, I, I, I, V, V, V, V],
             "llmrs_gather_rows": [V, I, V, I, V, I, V, I, I],
             "llmrs_combine_rows": [V, V, I, V, I, V, I, I, I],
+            "llmrs_expert_gemm_takes": [I, I],
+            "llmrs_expert_up": [V, V, I, I, V, V, V, I, ctypes.c_long, V, V, I, I, I, I, F, F],
+            "llmrs_expert_down": [V, V, I, V, V, I, ctypes.c_long, V, I, I, I],
+            "llmrs_expert_few_up": [V, V, I, I, V, V, I, I, V, I, I, I, I, F, F],
+            "llmrs_expert_few_down": [V, V, I, I, V, V, I, I, I, I, V, I],
             "llmrs_mingru_scan": [V, I, V, I, V, V, V, ctypes.c_long, V, V, I, I, V, I, I, V],
             "llmrs_causal_conv_silu": [V, I, V, I, V, V, V, ctypes.c_long, V, V, V, I, I, I, I, V, I],
             "llmrs_selective_scan": [V, I, V, I, V, I, I, I, V, I, V, V, V, V, I, V, ctypes.c_long, V, V, V, I, I, I, I, V, I, I, V],
@@ -280,6 +290,9 @@ class HipKernels(Kernels):
         if self.gemm_norms_whole(M, N, K):
             return NormPlan(True, 0)
         return None
+
+    def grouped_experts_take(self, hidden: int, ff: int, dtype: torch.dtype) -> bool:
+        return dtype == torch.bfloat16 and self.allow_mfma and bool(self.lib.llmrs_expert_gemm_takes(int(hidden), int(ff)))
 
     def gemm_defers_norm(self, M: int, N: int, K: int) -> bool:
         """Whether the bfloat16 product of M rows with an [N, K] weight takes `NormedRows` as its rows and, adding
@@ -871,6 +884,57 @@ class HipKernels(Kernels):
         assert row_token.dtype == row_of.dtype == torch.int32 and row_weight.dtype == torch.float32 and row_of.is_contiguous() and tuple(row_of.shape) == (T, E)
         self._run("route_rows", weights.numel() * 8, 0, None, self.lib.llmrs_route_rows, self._stream(), _p(weights), weights.stride(0), T, E,
                   _p(counts), _p(row_token), _p(row_weight), _p(row_of))
+
+    def expert_up(self, out: torch.Tensor, x: torch.Tensor, row_token: torch.Tensor, up: torch.Tensor, counts: torch.Tensor, row_weight: torch.Tensor,
+                  ff: int, activation: str, limit: float = 0.0, alpha: float = 1.0) -> None:
+        """out[r] = act(x[row_token[r]] Wup_e^T) * row_weight[r] for every row r of expert e, the experts' rows one after the
+        other, counts[e] of them (int32, on the device); `up` holds the experts' matrices one under the other (a gated
+        activation's gate and up rows in turn); out [rows, ff] in x's type, one rounding.  All experts in one launch."""
+        kind = {"relu2": 0, "clamped_glu": 1, "swiglu": 2}[activation]
+        E, K, rows = counts.numel(), x.shape[1], out.shape[0]
+        N = ff * (2 if kind else 1)
+        assert x.dtype == up.dtype == out.dtype == torch.bfloat16 and x.stride(1) == out.stride(1) == 1 and up.is_contiguous() and tuple(up.shape) == (E * N, K)
+        assert counts.dtype == row_token.dtype == torch.int32 and row_weight.dtype == torch.float32 and out.shape[1] == ff
+        assert row_token.numel() >= rows and row_weight.numel() >= rows and row_token.is_contiguous() and row_weight.is_contiguous()
+        self._run(f"expert_up {rows}x{N}x{K} of {E}", (rows * (K + ff) + E * N * K) * 2, 2 * rows * N * K, x.dtype, self.lib.llmrs_expert_up, self._stream(),
+                  _p(x), x.stride(0), x.shape[0], _p(row_token), _p(up), _p(counts), E, rows, _p(row_weight), _p(out), out.stride(0), int(ff), K, kind,
+                  float(limit), float(alpha))
+
+    def expert_down(self, y: torch.Tensor, a: torch.Tensor, down: torch.Tensor, counts: torch.Tensor) -> None:
+        """y[r] = a[r] Wdown_e^T in 32-bit for every row r of expert e (rows as for `expert_up`); `down` [hidden, experts * ff]
+        holds the experts' matrices side by side.  All experts in one launch."""
+        E, (rows, ff), D = counts.numel(), a.shape, down.shape[0]
+        assert a.dtype == down.dtype == torch.bfloat16 and y.dtype == torch.float32 and a.stride(1) == y.stride(1) == 1 and down.is_contiguous()
+        assert down.shape[1] == E * ff and tuple(y.shape) == (rows, D) and counts.dtype == torch.int32
+        self._run(f"expert_down {rows}x{D}x{ff} of {E}", (rows * ff + E * ff * D) * 2 + rows * D * 4, 2 * rows * D * ff, a.dtype, self.lib.llmrs_expert_down,
+                  self._stream(), _p(a), a.stride(0), _p(down), _p(counts), E, rows, _p(y), y.stride(0), D, ff)
+
+    def expert_few_up(self, out: torch.Tensor, x: torch.Tensor, up: torch.Tensor, weights: torch.Tensor, ff: int, activation: str, limit: float = 0.0,
+                      alpha: float = 1.0) -> None:
+        """For a step of up to 64 tokens: out[t, e * ff + f] = act(x[t] Wup_e^T)[f] * weights[t, e] (zero where weights is) for
+        every expert e that some token chose; the other experts' columns are not written, their matrices not read.  `up` as for
+        `expert_up`, weights float32 [T, experts]."""
+        kind = {"relu2": 0, "clamped_glu": 1, "swiglu": 2}[activation]
+        (T, E), K = weights.shape, x.shape[1]
+        N = ff * (2 if kind else 1)
+        assert x.dtype == up.dtype == out.dtype == torch.bfloat16 and x.stride(1) == out.stride(1) == weights.stride(1) == 1 and up.is_contiguous()
+        assert tuple(up.shape) == (E * N, K) and tuple(out.shape) == (T, E * ff) and x.shape[0] == T and weights.dtype == torch.float32
+        used = self._experts_used(weights)
+        self._run(f"expert_few_up {T}x{N}x{K} of {E}", (T * K + used * (N * K + T * ff)) * 2, 2 * T * used * N * K, x.dtype, self.lib.llmrs_expert_few_up, self._stream(),
+                  _p(x), x.stride(0), T, _p(up), _p(weights), weights.stride(0), E, _p(out), out.stride(0), int(ff), K, kind, float(limit), float(alpha))
+
+    def expert_few_down(self, h: torch.Tensor, act: torch.Tensor, down: torch.Tensor, weights: torch.Tensor) -> None:
+        """h[t] += sum over the experts that some token chose of act[t, expert's columns] Wdown_e^T; act as `expert_few_up` leaves
+        it, `down` as for `expert_down`."""
+        (T, E), D = weights.shape, h.shape[1]
+        assert act.dtype == down.dtype == torch.bfloat16 and h.dtype == weights.dtype == torch.float32 and down.is_contiguous()
+        assert act.stride(1) == h.stride(1) == weights.stride(1) == 1 and act.shape == (T, down.shape[1]) and h.shape[0] == T and down.shape == (D, act.shape[1])
+        ff, used = act.shape[1] // E, self._experts_used(weights)
+        self._run(f"expert_few_down {T}x{D}x{ff} of {E}", used * ff * (D + T) * 2 + T * D * 8, 2 * T * used * ff * D, act.dtype, self.lib.llmrs_expert_few_down,
+                  self._stream(), _p(act), act.stride(0), T, _p(down), _p(weights), weights.stride(0), E, ff, D, _p(h), h.stride(0))
+
+    def _experts_used(self, weights: torch.Tensor) -> int:
+        return int((weights != 0).any(0).sum().item()) if self.times is not None else 0      # (timing mode only: what a call reads)
 
     def gather_rows(self, out: torch.Tensor, x: torch.Tensor, rows: torch.Tensor) -> None:
         """out[r] = x[rows[r]]; rows int32."""

@@ -163,9 +163,17 @@ class RoutedFF(FeedForward):
     The experts' up matrices are laid one under the other and their down matrices side by side at load, so a step's
     experts are one up product of experts * intermediate_size columns, one pass that applies the activation and each
     column's expert weight (zero where the token did not choose the expert), and one down product: w_e Wdown_e act(.)
-    = Wdown_e (w_e act(.)).  A step with a prompt portion (never one that is recorded) whose experts would each get
-    `SORT_FROM_ROWS` rows or more on average lays the chosen (token, expert) pairs out expert by expert instead, and
-    every expert's rows are a product of their own: top / experts of the arithmetic.  The host reads how many tokens
+    = Wdown_e (w_e act(.)).
+
+    Steps of more than `GROUP_FROM_TOKENS` tokens lay the chosen (token, expert) pairs out expert by expert on the device and
+    run every expert's products over its own rows, all experts in one launch (`Kernels.expert_up`, `expert_down`): top /
+    experts of the arithmetic, the activation and the expert's weight in the first product's epilogue.  Steps of up to
+    `FEW_TOKENS` tokens, or of so few that they cannot choose every expert, run the product over all experts in kernels that
+    leave the experts that no token chose unread (`expert_few_up`, `expert_few_down`).  Both are for bfloat16 and sizes those kernels take (`Kernels.grouped_experts_take`).
+
+    Elsewhere a step with a prompt portion (never one that is recorded) whose experts would each get
+    `SORT_FROM_ROWS` rows or more on average lays the pairs out in the same way, and
+    every expert's rows are an ordinary product of their own.  The host reads how many tokens
     each expert got (one small copy) to size those products; the down matrices are kept a second time, one by one.
     That is for experts whose matrices have `SORT_FROM_WEIGHT` elements or more: the products of smaller experts over
     a few hundred rows each leave most of the device idle, and the one product over all experts, four times the
@@ -181,6 +189,10 @@ class RoutedFF(FeedForward):
     equal groups of neighbours, and only those of the `keep` groups whose best expert is best can be chosen; `shared` = {kind, prefix leaf, params}: a
     feed-forward of any registered kind that every token passes beside its experts, added in."""
     graph_safe = True
+    GROUP_FROM_TOKENS = 64          # (the kernels for few tokens take no more)
+    # 16 experts of 2048 x 2048 of which 4, against the one product over all of them: 1 token 50 against 92 us, 4 73 against 100,
+    # 8 109 against 104, 16 123 against 116 (all experts chosen), 32 180 against 115; grouped from 65 tokens on 141 against 153
+    FEW_TOKENS = 16
     SORT_FROM_ROWS = 128
     SORT_FROM_WEIGHT = 8 << 20
 
@@ -223,6 +235,7 @@ class RoutedFF(FeedForward):
         self.w_router = self.w_up = self.w_down = self.w_down_each = self.correction = None
         shared = p.get("shared")
         self.shared = None
+        self.grouped = False            # whether the kernels run all experts over their own rows in one launch
         if shared is not None:
             from ..config.spec import PartSpec
             self.shared = build_feed_forward(PartSpec(shared["kind"], self.name(shared["prefix"]), dict(shared["params"])), dtype)
@@ -254,9 +267,12 @@ class RoutedFF(FeedForward):
         else:
             self.w_up = torch.cat([get(n) for n in self.n_up], dim=0).contiguous()
         self.w_down = torch.cat([place(tensors[n], device, self.dtype) for n in self.n_down], dim=1).contiguous()
-        # each expert's down matrix by itself, for the steps that run the experts one by one (not when all are chosen)
+        # each expert's down matrix by itself, for the steps that run the experts one by one (not when all are chosen, nor
+        # where the grouped products run)
+        on_device = torch.device(device).type == "cuda" or stand_in_kernels()
+        self.grouped = self.top < self.experts and on_device and kernels().grouped_experts_take(self.hidden, self.inter, self.dtype)
         self.w_down_each = (self.w_down.view(self.hidden, self.experts, self.inter).permute(1, 0, 2).contiguous()
-                            if self.top < self.experts and self.inter * self.hidden >= self.SORT_FROM_WEIGHT else None)
+                            if self.top < self.experts and not self.grouped and self.inter * self.hidden >= self.SORT_FROM_WEIGHT else None)
 
     def export(self):
         up, down = self.w_up.cpu(), self.w_down.cpu()
@@ -297,6 +313,13 @@ class RoutedFF(FeedForward):
             k.route_topk(logits, weights, self.top, self.renormalize, **groups)
         if self.shared is not None:         # (reads x, adds into h; the experts' buffers are its own until it is done)
             self.shared.forward(ctx, x, h)
+        if self.grouped and T > self.GROUP_FROM_TOKENS:
+            return self._forward_grouped(ctx, x, h, weights)
+        if self.grouped and T <= self.GROUP_FROM_TOKENS and (T <= self.FEW_TOKENS or T * self.top < self.experts):
+            act = ctx.workspace("mlp.act", (T, N), self.dtype)
+            k.expert_few_up(act, x, self.w_up, weights, self.inter, self.activation, self.limit, self.alpha)
+            k.expert_few_down(h, act, self.w_down, weights)
+            return ctx.note_left(h, None)
         if (self.w_down_each is not None and ctx.longest > 1 and T * self.top >= self.SORT_FROM_ROWS * self.experts
                 and self.inter * self.hidden >= self.SORT_FROM_WEIGHT):
             return self._forward_sorted(ctx, x, h, weights)
@@ -307,20 +330,39 @@ class RoutedFF(FeedForward):
         k.gemm(act, self.w_down, h, EPI_ACCUM_F32, ctx.gemm_workspace(act, self.w_down))
         ctx.note_left(h, None)
 
-
-    def _forward_sorted(self, ctx, x, h, weights):
+    def _rows_by_expert(self, ctx, weights):
+        """The step's (token, expert) pairs expert by expert, on the device: how many rows each expert has, each row's token
+        and weight, and where a token's rows lie.  (A chosen expert whose score is exactly zero has no row: it adds nothing.)"""
         k = kernels()
-        T, E, F, D = x.shape[0], self.experts, self.inter, self.hidden
+        T, E = weights.shape
         rows = T * self.top
         counts = ctx.workspace("moe.counts", (E,), torch.int32)
         k.route_counts(weights, counts)
-        n_of = counts.cpu().tolist()                 # (the step waits here: the experts' products are sized by these)
-        total = sum(n_of)                            # (a chosen expert whose score is exactly zero has no row: it adds nothing)
-        assert total <= rows
         row_token = ctx.workspace("moe.row_token", (rows,), torch.int32)
         row_weight = ctx.workspace("moe.row_weight", (rows, 1), torch.float32)
         row_of = ctx.workspace("moe.row_of", (T, E), torch.int32)
         k.route_rows(weights, counts, row_token, row_weight, row_of)
+        return counts, row_token, row_weight, row_of
+
+    def _forward_grouped(self, ctx, x, h, weights):
+        k = kernels()
+        counts, row_token, row_weight, row_of = self._rows_by_expert(ctx, weights)
+        rows = row_token.shape[0]
+        act = ctx.workspace("mlp.act", (rows, self.inter), self.dtype)
+        k.expert_up(act, x, row_token, self.w_up, counts, row_weight, self.inter, self.activation, self.limit, self.alpha)
+        ys = ctx.workspace("moe.y", (rows, self.hidden), torch.float32)
+        k.expert_down(ys, act, self.w_down, counts)
+        k.combine_rows(h, ys, row_of)
+        ctx.note_left(h, None)
+
+    def _forward_sorted(self, ctx, x, h, weights):
+        k = kernels()
+        T, E, F, D = x.shape[0], self.experts, self.inter, self.hidden
+        counts, row_token, row_weight, row_of = self._rows_by_expert(ctx, weights)
+        rows = row_token.shape[0]
+        n_of = counts.cpu().tolist()                 # (the step waits here: the experts' products are sized by these)
+        total = sum(n_of)
+        assert total <= rows
         if total == 0:
             return ctx.note_left(h, None)
         xs = ctx.workspace("moe.x", (rows, D), self.dtype)[:total]

@@ -156,6 +156,71 @@ def test_two_maps_are_finished_into_one_row_of_keys(H, G, d, dv, T, dtype):
     close(vc.cpu()[at, :, :, off], s[:, 2 * (H + G) * d:-1].reshape(T, G, dv), dt, "values")
 
 
+def plain_expert_sum(x, t, weights, E, act, limit, alpha):
+    """sum_e weights[:, e] Wdown_e act(..), from the part's tensors."""
+    out = torch.zeros_like(x)
+    for e in range(E):
+        u = x @ t[f"x.experts.{e}.up_proj.weight"].double().T
+        if act == "relu2":
+            a = torch.clamp(u, min=0.0) ** 2
+        else:
+            g = x @ t[f"x.experts.{e}.gate_proj.weight"].double().T
+            if act == "swiglu":
+                a = g / (1.0 + torch.exp(-g)) * u
+            else:
+                g, u = torch.clamp(g, max=limit), torch.clamp(u, min=-limit, max=limit)
+                a = g / (1.0 + torch.exp(-alpha * g)) * (u + 1.0)
+        out += (a * weights[:, e:e + 1]) @ t[f"x.experts.{e}.down_proj.weight"].double().T
+    return out
+
+
+@pytest.mark.parametrize("act", ["swiglu", "clamped_glu", "relu2"])
+@pytest.mark.parametrize("E,top,D,F", [(5, 2, 64, 64), (16, 4, 320, 128), (70, 3, 192, 64), (12, 1, 128, 192), (3, 2, 640, 320)])
+def test_experts_over_their_own_rows(E, top, D, F, act):
+    """The products over the rows that chose each expert (grouped tiles) and those of steps of few tokens that leave unchosen
+    experts unread, at token counts around every kernel's bounds, against plain tensor code; an expert that nobody chose, one
+    that everybody chose, weights of exactly zero."""
+    k = kernels()
+    g = torch.Generator().manual_seed(E + F)
+    n_up = F if act == "relu2" else 2 * F
+    up, down = (torch.randn(E, n_up, D, generator=g) * 0.1).to(torch.bfloat16), (torch.randn(E, D, F, generator=g) * 0.1).to(torch.bfloat16)
+    t = {}
+    for e in range(E):
+        t[f"x.experts.{e}.up_proj.weight"] = up[e] if act == "relu2" else up[e][1::2]
+        t[f"x.experts.{e}.gate_proj.weight"] = up[e][0::2]
+        t[f"x.experts.{e}.down_proj.weight"] = down[e]
+    assert k.grouped_experts_take(D, F, torch.bfloat16) and not k.grouped_experts_take(D + 8, F, torch.bfloat16) and not k.grouped_experts_take(D, F, torch.float32)
+    w_up, w_down = up.reshape(E * n_up, D).cuda(), down.permute(1, 0, 2).reshape(D, E * F).contiguous().cuda()
+    for T in (1, 3, 4, 5, 16, 17, 33, 64, 65, 130, 257, 400):
+        x = torch.randn(T, D, generator=g).to(torch.bfloat16)
+        weights = torch.zeros(T, E)
+        choice = torch.rand(T, E, generator=g)
+        choice[:, 0] = 2.0 if top > 1 else choice[:, 0]          # everybody's
+        choice[:, E - 1] = -1.0                                   # nobody's
+        weights.scatter_(1, choice.topk(top, dim=1).indices, 0.1 + torch.rand(T, top, generator=g))
+        weights[T // 2] = 0.0
+        h = torch.randn(T, D, generator=g)
+        want = plain_expert_sum(x.double(), t, weights.double(), E, act, 1.5, 1.702)
+        wd, xd = weights.cuda(), x.cuda()
+        if T <= 64:
+            hd = h.cuda()
+            a = torch.full((T, E * F), float("nan"), dtype=torch.bfloat16, device="cuda")
+            k.expert_few_up(a, xd, w_up, wd, F, act, 1.5, 1.702)
+            k.expert_few_down(hd, a, w_down, wd)
+            close(hd.cpu() - h, want, torch.bfloat16, f"few, {T} tokens")
+        hd, rows = h.cuda(), T * top
+        counts, row_of = torch.empty(E, dtype=torch.int32, device="cuda"), torch.empty(T, E, dtype=torch.int32, device="cuda")
+        row_token, row_weight = torch.empty(rows, dtype=torch.int32, device="cuda"), torch.empty(rows, 1, device="cuda")
+        k.route_counts(wd, counts)
+        assert counts.tolist() == (weights > 0).sum(0).tolist()
+        k.route_rows(wd, counts, row_token, row_weight, row_of)
+        a, y = torch.empty(rows, F, dtype=torch.bfloat16, device="cuda"), torch.empty(rows, D, device="cuda")
+        k.expert_up(a, xd, row_token, w_up, counts, row_weight, F, act, 1.5, 1.702)
+        k.expert_down(y, a, w_down, counts)
+        k.combine_rows(hd, y, row_of)
+        close(hd.cpu() - h, want, torch.bfloat16, f"grouped, {T} tokens")
+
+
 class Paged:
     """Random keys and values of several requests, in pages handed out in random order."""
 
